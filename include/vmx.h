@@ -1297,6 +1297,115 @@ int vmx_gezozen_forward(vmx_gezozen *m, const int32_t *tokens, const int32_t *po
                         const int32_t *state_slots, const int32_t *logit_rows, int num_logit_rows, float *logits, int32_t *greedy_ids,
                         float *layer_trace, void *stream);
 
+/* ------------------------------------------------- latent queries, exponential-gate memory, corrected router, Fofinex executor */
+
+/* What vmx_latent_prepare_rows does to a step's f32 rows; a part whose input pointer is NULL is skipped. */
+typedef struct vmx_latent_prepare {
+    const float *kv;              /* rows [kv_rank | rot_dim]: the first part RMS-normed, the second rotated, both to cache row slots[t] */
+    int64_t ldkv;
+    const uint16_t *latent_norm_bf16;   /* gain of the normed latent [kv_rank] */
+    const float *q;               /* query rows, per head [dim | rot_dim]: the rotated parts go to q_rot [tokens, heads, rot_dim] */
+    int64_t ldq;
+    int heads, dim;
+    float *q_rot;
+    const float *q_latent;        /* rows of q_rank numbers, RMS-normed to q_latent_out [tokens, q_rank] */
+    int64_t ldq_latent;
+    int q_rank;
+    const uint16_t *q_latent_norm_bf16;
+    int kv_rank, rot_dim;
+    float eps;
+    const float *inv_freq;        /* angle step per pair [rot_dims / 2] */
+    int rot_dims;                 /* rotated coordinates of the rot_dim (the rest pass unchanged) */
+    int rot_halves;               /* coordinate i turns with i + rot_dims / 2 instead of 2i with 2i + 1 */
+    float rot_mul;                /* cos and sin are multiplied by this (0: 1) */
+} vmx_latent_prepare;
+/* The parts of vmx_latent_kv_prepare one by one, for layers whose queries come through a latent of their own (two calls, the
+ * query product between them) or that attend over another layer's cache (no kv).  cache_dtype (VMX_F32 / VMX_BF16) is the element
+ * type of the cache and of q_latent_out; a negative slot is not stored. */
+int vmx_latent_prepare_rows(const vmx_latent_prepare *prep, const int32_t *positions, const int32_t *slots, void *cache, int cache_dtype,
+                            void *q_latent_out, int tokens, void *stream);
+
+/* vmx_matrix_memory_recurrence with a write gain and a normaliser. */
+typedef struct vmx_matrix_memory_opts {
+    const float *write_gain;      /* [tokens, ldgain] per head: the plain write is S <- g S + gain k v^T (beta NULL) */
+    int64_t ldgain;
+    float *norm_out;              /* [tokens, ldnorm] per head: n . q with n <- g n + gain k carried beside S (NULL: none); the state then */
+    int64_t ldnorm;               /* has vdim + 1 columns: vmx_gated_delta_rule_state_bytes(slots, heads, dim, vdim + 1) */
+} vmx_matrix_memory_opts;
+int vmx_matrix_memory_recurrence_ex(float *o, int64_t ldo, const float *q, int64_t ldq, float q_mul, const float *k, int64_t ldk,
+                                    const float *v, int64_t ldv, const float *g, int64_t ldg, int g_per_head, const float *beta,
+                                    int64_t ldbeta, float *state, const int32_t *positions, const int32_t *seq_starts,
+                                    const int32_t *state_slots, int num_seqs, int heads, int qk_heads, int dim, int vdim,
+                                    const vmx_matrix_memory_opts *opts, void *stream);
+/* Gates of a memory with an exponential input gate, in place: with i = cap tanh(input / cap), f = log(sigmoid(cap tanh(forget / cap)))
+ * and the running maximum m_t = max(f_t + m_(t-1), i_t) per head (0 before position 0; kept in max_state [slots, heads]), input <-
+ * exp(i_t - m_t) (the write gain), forget <- exp(f_t + m_(t-1) - m_t) (the decay), floor <- exp(-m_t). */
+int vmx_exp_gate_scan(float *input_gate, int64_t ldi, float *forget_gate, int64_t ldf, float *floor, int64_t ldfloor, float *max_state,
+                      float cap, const int32_t *positions, const int32_t *seq_starts, const int32_t *state_slots, int num_seqs, int heads,
+                      void *stream);
+/* vmx_head_rms_gate with its options open. */
+typedef struct vmx_read_out_opts {
+    int gate_silu;                /* y *= gate * sigmoid(gate) instead of sigmoid(gate) */
+    int w_per_head;               /* the gain holds heads * vdim numbers instead of vdim shared ones */
+    const float *norm;            /* not NULL: o[t, h] is divided by max(|norm[t, h]|, floor[t, h]) + norm_eps before the RMS norm */
+    int64_t ldnorm;
+    const float *floor;
+    int64_t ldfloor;
+    float norm_eps;
+} vmx_read_out_opts;
+int vmx_head_read_out(void *y, int y_dtype, const float *o, int64_t ldo, const uint16_t *w_bf16, const float *gate, int64_t ldgate,
+                      float eps, int tokens, int heads, int vdim, const vmx_read_out_opts *opts, void *stream);
+
+/* Group-limited choice over corrected sigmoid scores: score = sigmoid(logit), choice score = score + correction (bf16 per expert);
+ * a group's score is the sum of its two largest choice scores, only experts of the keep_groups best groups can be chosen, k rounds
+ * of argmax over the choice scores (ties -> smaller index).  weights = the chosen experts' scores (without the correction) * scale.
+ * Logits rows are ld_logits numbers apart. */
+int vmx_grouped_topk_sigmoid(const float *logits, int64_t ld_logits, const uint16_t *correction_bf16, float *topk_weights,
+                             int32_t *topk_ids, int tokens, int num_experts, int k, int groups, int keep_groups, float scale, void *stream);
+
+#define VMX_MIXER_EXP_MEMORY 8           /* matrix memory with exponential input gate, forget gate, normaliser and running maximum */
+#define VMX_MLP_DENSE_GLU 6              /* biased gate / up / down, tanh-form gelu */
+#define VMX_MLP_CORRECTED_MOE 7          /* corrected sigmoid scores, group-limited; squared-ReLU experts + gated shared expert */
+
+/* One layer of a Fofinex model: x <- x + N1b(mixer(N1(x))); x <- x + N2b(ff(N2(x))), N a layer norm with a gain. */
+typedef struct vmx_fofinex_layer_config {
+    int mixer;                    /* VMX_MIXER_LATENT_ATTENTION or VMX_MIXER_EXP_MEMORY */
+    int heads, dim, vdim;         /* latent attention: dim unrotated query/key coordinates; memory: key size */
+    int rot_dim, kv_rank, q_rank; /* latent attention: rotated coordinates, key/value and query latent sizes */
+    float scale;                  /* latent attention: score scale */
+    vmx_rotation rot;             /* latent attention: rotation in halves of the rot_dim part (dims 0: none) */
+    int kv_from;                  /* latent attention: the earlier layer whose cache it attends over (-1: its own) */
+    float gate_cap;               /* memory: cap of both gates' logits */
+    int mlp;                      /* VMX_MLP_NONE, VMX_MLP_DENSE_GLU or VMX_MLP_CORRECTED_MOE */
+    int ff;                       /* dense */
+    int experts, top, groups, keep_groups, expert_ff, shared_ff;   /* shared_ff 0: no shared expert */
+    float router_scale;
+} vmx_fofinex_layer_config;
+
+typedef struct vmx_fofinex_config {
+    int vocab, width, num_layers;
+    float norm_eps;
+    int dtype;                    /* VMX_BF16: bf16 operands and cache; VMX_F32: everything in f32 */
+    int block_size, num_blocks;   /* paged latent cache: rows per block, blocks per layer */
+    int max_tokens, max_seqs;     /* most tokens / sequences of one forward call */
+    int state_slots;              /* recurrent-state slots (one per live sequence) */
+} vmx_fofinex_config;
+
+typedef struct vmx_fofinex vmx_fofinex;
+int vmx_fofinex_create(const vmx_fofinex_config *cfg, const vmx_fofinex_layer_config *layers, vmx_fofinex **out);
+void vmx_fofinex_destroy(vmx_fofinex *m);
+/* One checkpoint tensor under its name in the file: "embed" (also the output matrix), "embed.norm", "final.norm",
+ * "l<i>.norm1|norm1b|norm2|norm2b"; latent attention "l<i>.mix.dq|dq.norm|uq|dkv|dkv.norm|uk|uv|o"; memory
+ * "l<i>.mix.q|k|v|g|o|norm|i|i.b|f|f.b"; dense "l<i>.mlp.gate|up|down" (+ ".b"); mixture "l<i>.mlp.router|correction",
+ * "l<i>.mlp.e<j>.up|down", "l<i>.mlp.shared.up|down|sg": bf16, matrices [out, in]; host or device memory. */
+int vmx_fofinex_load_tensor(vmx_fofinex *m, const char *name, const void *data, size_t bytes, void *stream);
+int vmx_fofinex_missing_tensors(const vmx_fofinex *m);
+/* One step over packed tokens, arguments as vmx_gupuvik_forward. */
+int vmx_fofinex_forward(vmx_fofinex *m, const int32_t *tokens, const int32_t *positions, const int32_t *slots, const int32_t *seq_ids,
+                        int num_tokens, const int32_t *block_tables, int num_seqs, int max_blocks_per_seq, const int32_t *seq_starts,
+                        const int32_t *state_slots, const int32_t *logit_rows, int num_logit_rows, float *logits, int32_t *greedy_ids,
+                        float *layer_trace, void *stream);
+
 #ifdef __cplusplus
 }
 #endif

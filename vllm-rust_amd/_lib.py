@@ -257,6 +257,16 @@ _SIGS = {
     "vmx_gezozen_load_tensor": (_i, [_p, C.c_char_p, _p, _sz, _p]),
     "vmx_gezozen_missing_tensors": (_i, [_p]),
     "vmx_gezozen_forward": (_i, [_p, _p, _p, _p, _p, _i, _p, _i, _i, _p, _p, _p, _i, _p, _p, _p, _p]),
+    "vmx_latent_prepare_rows": (_i, [_p, _p, _p, _p, _i, _p, _i, _p]),
+    "vmx_matrix_memory_recurrence_ex": (_i, [_p, _i64, _p, _i64, _f, _p, _i64, _p, _i64, _p, _i64, _i, _p, _i64, _p, _p, _p, _p, _i, _i, _i, _i, _i, _p, _p]),
+    "vmx_exp_gate_scan": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _f, _p, _p, _p, _i, _i, _p]),
+    "vmx_head_read_out": (_i, [_p, _i, _p, _i64, _p, _p, _i64, _f, _i, _i, _i, _p, _p]),
+    "vmx_grouped_topk_sigmoid": (_i, [_p, _i64, _p, _p, _p, _i, _i, _i, _i, _i, _f, _p]),
+    "vmx_fofinex_create": (_i, [_p, _p, _p]),
+    "vmx_fofinex_destroy": (None, [_p]),
+    "vmx_fofinex_load_tensor": (_i, [_p, C.c_char_p, _p, _sz, _p]),
+    "vmx_fofinex_missing_tensors": (_i, [_p]),
+    "vmx_fofinex_forward": (_i, [_p, _p, _p, _p, _p, _i, _p, _i, _i, _p, _p, _p, _i, _p, _p, _p, _p]),
 }
 
 
@@ -373,8 +383,44 @@ class GezozenConfig(C.Structure):
     ]
 
 
+class LatentPrepare(C.Structure):
+    """struct vmx_latent_prepare (include/vmx.h)."""
+    _fields_ = [
+        ("kv", _p), ("ldkv", _i64), ("latent_norm_bf16", _p), ("q", _p), ("ldq", _i64), ("heads", _i), ("dim", _i), ("q_rot", _p),
+        ("q_latent", _p), ("ldq_latent", _i64), ("q_rank", _i), ("q_latent_norm_bf16", _p), ("kv_rank", _i), ("rot_dim", _i), ("eps", _f),
+        ("inv_freq", _p), ("rot_dims", _i), ("rot_halves", _i), ("rot_mul", _f),
+    ]
+
+
+class MatrixMemoryOpts(C.Structure):
+    """struct vmx_matrix_memory_opts (include/vmx.h)."""
+    _fields_ = [("write_gain", _p), ("ldgain", _i64), ("norm_out", _p), ("ldnorm", _i64)]
+
+
+class ReadOutOpts(C.Structure):
+    """struct vmx_read_out_opts (include/vmx.h)."""
+    _fields_ = [("gate_silu", _i), ("w_per_head", _i), ("norm", _p), ("ldnorm", _i64), ("floor", _p), ("ldfloor", _i64), ("norm_eps", _f)]
+
+
+class FofinexLayerConfig(C.Structure):
+    """struct vmx_fofinex_layer_config (include/vmx.h)."""
+    _fields_ = [
+        ("mixer", _i), ("heads", _i), ("dim", _i), ("vdim", _i), ("rot_dim", _i), ("kv_rank", _i), ("q_rank", _i), ("scale", _f),
+        ("rot", Rotation), ("kv_from", _i), ("gate_cap", _f), ("mlp", _i), ("ff", _i), ("experts", _i), ("top", _i), ("groups", _i),
+        ("keep_groups", _i), ("expert_ff", _i), ("shared_ff", _i), ("router_scale", _f),
+    ]
+
+
+class FofinexConfig(C.Structure):
+    """struct vmx_fofinex_config (include/vmx.h)."""
+    _fields_ = [
+        ("vocab", _i), ("width", _i), ("num_layers", _i), ("norm_eps", _f), ("dtype", _i), ("block_size", _i), ("num_blocks", _i),
+        ("max_tokens", _i), ("max_seqs", _i), ("state_slots", _i),
+    ]
+
+
 # one-family libraries (csrc/Makefile FAMILY=...): the entry points of the other families are absent and stay unbound
-FAMILY_LIBS = ("vokepel", "gezozen")
+FAMILY_LIBS = ("vokepel", "gezozen", "fofinex")
 
 
 def _bind():

@@ -12,11 +12,18 @@
 //   S <- diag(g_t) S;   u = beta_t (v_t - S^T k_t);   S <- S + k_t u^T;   o_t = S^T q_t
 // so a token reads the memory after its own write (computed as (g S)^T q + u (k . q), the same sum in another order).  The decay
 // g_t is a number per key channel, or one per head (per token, or a constant of the head: row stride 0); without beta the write
-// is the plain outer product, u = v_t (S <- diag(g_t) S + k_t v_t^T: gated linear attention, retention).  Query/key
+// is the plain outer product, u = v_t (S <- diag(g_t) S + k_t v_t^T: gated linear attention, retention), optionally times a number
+// per head and token (the write gain of a memory with an input gate).  A NORMALISER may ride along as one more value column that
+// is 1 for every token: n <- g n + gain k, read out as n . q per head.  Query/key
 // head of value head h: h / (heads / qk_heads).  A workgroup owns 16 value columns of one (sequence, head) and walks the
 // sequence's tokens of the step in order; 16 threads share a column, each holding every 16th row of S in registers, and the
 // column sums per token are 16-lane butterflies.  The state slot keeps S in the workgroup's own register order (the layout is
 // private to this kernel), so that loading and storing it is coalesced.
+//
+// Exponential gates (vmx_exp_gate_scan): a memory whose input gate is an exponential keeps the logarithm of its scale, a running
+// maximum m_t = max(f_t + m_(t-1), i_t) per head (from 0), in its slot; what the recurrence needs are the decay
+// exp(f_t + m_(t-1) - m_t), the write gain exp(i_t - m_t) and, for the read-out, exp(-m_t).  The maximum is a prefix scan over
+// (sum of f, largest of "i plus the f after it") pairs: one wave per (sequence, head), 64 tokens a round.
 #include "vmx_kernels.h"
 
 namespace {
@@ -134,8 +141,10 @@ struct DeltaArgs {
     const int32_t *positions, *seq_starts, *state_slots;
     int heads, qk_heads, dim, vdim;
     int g_per_head;                          // g rows hold one decay per head (ldg 0: the same row for every token) instead of heads * dim
-    int plain;                               // no beta: u = v
+    int plain;                               // u = beta v (beta NULL: u = v) instead of beta (v - S^T k)
     float q_mul;                             // the queries are multiplied by this constant as they are read
+    float *norm;                             // [tokens, ldnorm] n . q per head: value column vdim is 1 for every token (NULL: no such column)
+    int64_t ldnorm;
 };
 
 constexpr int DR_RS = 16, DR_VT = 16;   // row splits per column, columns per workgroup
@@ -179,9 +188,9 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(const DeltaArgs a
 #pragma unroll
         for (int j = 0; j < NV; j++) {
             const int i = tid + 256 * j, tt = i / DR_VT, cc = tile * DR_VT + i % DR_VT;
-            rv[j] = (tt < ct && cc < a.vdim) ? a.v[(int64_t)(first + t0 + tt) * a.ldv + (int64_t)h * a.vdim + cc] : 0.f;
+            rv[j] = (tt < ct && cc < a.vdim) ? a.v[(int64_t)(first + t0 + tt) * a.ldv + (int64_t)h * a.vdim + cc] : (cc == a.vdim && a.norm ? 1.f : 0.f);
         }
-        rb = (tid < ct && !a.plain) ? a.beta[(int64_t)(first + t0 + tid) * a.ldbeta + h] : 0.f;
+        rb = (tid < ct && a.beta) ? a.beta[(int64_t)(first + t0 + tid) * a.ldbeta + h] : 1.f;
     };
     auto stage = [&](int b) {
 #pragma unroll
@@ -235,8 +244,11 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(const DeltaArgs a
             pk += vmx_dpp<VMX_DPP_XOR2>(pk), pq += vmx_dpp<VMX_DPP_XOR2>(pq), kq += vmx_dpp<VMX_DPP_XOR2>(kq);
             pk += vmx_dpp<VMX_DPP_HALF_MIRROR>(pk), pq += vmx_dpp<VMX_DPP_HALF_MIRROR>(pq), kq += vmx_dpp<VMX_DPP_HALF_MIRROR>(kq);
             pk += vmx_dpp<VMX_DPP_ROR8>(pk), pq += vmx_dpp<VMX_DPP_ROR8>(pq), kq += vmx_dpp<VMX_DPP_ROR8>(kq);
-            const float uu = a.plain ? vv : bv * (vv - pk);
-            if (r == 0 && c < a.vdim) a.o[(int64_t)(first + t0 + tt) * a.ldo + (int64_t)h * a.vdim + c] = fmaf(uu, kq, pq);
+            const float uu = bv * (a.plain ? vv : vv - pk);
+            if (r == 0) {
+                if (c < a.vdim) a.o[(int64_t)(first + t0 + tt) * a.ldo + (int64_t)h * a.vdim + c] = fmaf(uu, kq, pq);
+                else if (c == a.vdim && a.norm) a.norm[(int64_t)(first + t0 + tt) * a.ldnorm + h] = fmaf(uu, kq, pq);
+            }
 #pragma unroll
             for (int u = 0; u < DPT; u++) S[u] = fmaf(kk[u], uu, S[u]);
         };
@@ -257,19 +269,63 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(const DeltaArgs a
     for (int u = 0; u < DPT; u++) sp[(int64_t)u * 256] = S[u];
 }
 
+// In place, one wave per (sequence, head): i[t, h] <- exp(i_t - m_t), f[t, h] <- exp(f_t + m_(t-1) - m_t), floor[t, h] = exp(-m_t)
+// with i_t = cap tanh(i / cap), f_t = log(sigmoid(cap tanh(f / cap))) and m the running maximum (the slot's; 0 at position 0).
+__global__ __launch_bounds__(64) void exp_gate_scan_kernel(float *__restrict__ ig, int64_t ldi, float *__restrict__ fg, int64_t ldf,
+                                                            float *__restrict__ floor, int64_t ldfloor, float *__restrict__ m_state, float cap,
+                                                            const int32_t *__restrict__ positions, const int32_t *__restrict__ seq_starts,
+                                                            const int32_t *__restrict__ state_slots, int heads) {
+    const int h = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x;
+    const int first = seq_starts[seq], count = seq_starts[seq + 1] - first;
+    if (count <= 0) return;
+    float *ms = m_state + (int64_t)state_slots[seq] * heads + h;
+    float m0 = positions[first] == 0 ? 0.f : *ms;
+    for (int t0 = 0; t0 < count; t0 += 64) {
+        const bool in = t0 + lane < count;
+        const int64_t row = first + t0 + lane;
+        const float li = in ? cap * tanhf(ig[row * ldi + h] / cap) : -1e30f;
+        const float lf = in ? -softplus_f(-cap * tanhf(fg[row * ldf + h] / cap)) : 0.f;
+        float A = lf, B = li;      // over the tokens of this round up to this lane's: sum of f; largest i plus the f after it
+#pragma unroll
+        for (int d = 1; d < 64; d <<= 1) {
+            const float pa = __shfl_up(A, d, 64), pb = __shfl_up(B, d, 64);
+            if (lane >= d) {
+                B = fmaxf(pb + A, B);
+                A += pa;
+            }
+        }
+        const float m = fmaxf(m0 + A, B), up = __shfl_up(m, 1, 64), prev = lane == 0 ? m0 : up;
+        if (in) {
+            ig[row * ldi + h] = expf(li - m);
+            fg[row * ldf + h] = expf(lf + prev - m);
+            floor[row * ldfloor + h] = expf(-m);
+        }
+        m0 = __shfl(m, min(63, count - t0 - 1), 64);
+    }
+    if (lane == 0) *ms = m0;
+}
+
 // y[t, h] = o[t, h] / sqrt(mean(o^2) + eps) * w * sigmoid(gate[t, h]) (gate_silu: * silu(gate[t, h])); one wave per (token, head);
-// w bf16 [vdim] shared by heads (NULL: no gain)
+// w bf16 [vdim] shared by heads or (w_per_head) [heads * vdim] (NULL: no gain).  norm != NULL: o is divided by
+// max(|norm[t, h]|, floor[t, h]) + norm_eps first.
 __global__ __launch_bounds__(256) void head_rms_gate_kernel(void *__restrict__ y, int y_f32, const float *__restrict__ o, int64_t ldo,
                                                              const uint16_t *__restrict__ w, const float *__restrict__ gate, int64_t ldgate,
-                                                             float eps, int rows, int heads, int vdim, int gate_silu) {
+                                                             float eps, int rows, int heads, int vdim, int gate_silu, int w_per_head,
+                                                             const float *__restrict__ norm, int64_t ldnorm, const float *__restrict__ floor,
+                                                             int64_t ldfloor, float norm_eps) {
     const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (row >= rows) return;
     const int t = row / heads, h = row % heads;
     const float *src = o + (int64_t)t * ldo + (int64_t)h * vdim;
+    if (w && w_per_head) w += (int64_t)h * vdim;
+    const float div = norm ? 1.0f / (fmaxf(fabsf(norm[(int64_t)t * ldnorm + h]), floor[(int64_t)t * ldfloor + h]) + norm_eps) : 1.0f;
     float ss = 0.f;
-    for (int i = lane; i < vdim; i += 64) ss = fmaf(src[i], src[i], ss);
+    for (int i = lane; i < vdim; i += 64) {
+        const float v = src[i] * div;
+        ss = fmaf(v, v, ss);
+    }
     ss = vmx_wave_sum(ss);
-    const float inv = 1.0f / sqrtf(ss / (float)vdim + eps);
+    const float inv = div / sqrtf(ss / (float)vdim + eps);
     for (int i = lane; i < vdim; i += 64) {
         float v = src[i] * inv;
         if (w) v *= vmx_bf16_to_f32(w[i]);
@@ -377,15 +433,28 @@ extern "C" int vmx_matrix_memory_recurrence(float *o, int64_t ldo, const float *
                                             int64_t ldv, const float *g, int64_t ldg, int g_per_head, const float *beta, int64_t ldbeta,
                                             float *state, const int32_t *positions, const int32_t *seq_starts, const int32_t *state_slots,
                                             int num_seqs, int heads, int qk_heads, int dim, int vdim, void *stream) {
+    return vmx_matrix_memory_recurrence_ex(o, ldo, q, ldq, q_mul, k, ldk, v, ldv, g, ldg, g_per_head, beta, ldbeta, state, positions, seq_starts,
+                                           state_slots, num_seqs, heads, qk_heads, dim, vdim, nullptr, stream);
+}
+
+extern "C" int vmx_matrix_memory_recurrence_ex(float *o, int64_t ldo, const float *q, int64_t ldq, float q_mul, const float *k, int64_t ldk,
+                                               const float *v, int64_t ldv, const float *g, int64_t ldg, int g_per_head, const float *beta,
+                                               int64_t ldbeta, float *state, const int32_t *positions, const int32_t *seq_starts,
+                                               const int32_t *state_slots, int num_seqs, int heads, int qk_heads, int dim, int vdim,
+                                               const vmx_matrix_memory_opts *opts, void *stream) {
     VMX_REQUIRE(o && q && k && v && g && state && positions && seq_starts && state_slots, "matrix_memory_recurrence: null pointer");
     VMX_REQUIRE(heads >= 1 && qk_heads >= 1 && heads % qk_heads == 0, "matrix_memory_recurrence: %d heads do not share %d query/key heads evenly",
                 heads, qk_heads);
     VMX_REQUIRE(dim >= 1 && dim <= 256 && vdim >= 1, "matrix_memory_recurrence: key size %d outside 1..256", dim);
     VMX_REQUIRE(ldg >= (g_per_head ? heads : (int64_t)heads * dim) || (g_per_head && ldg == 0), "matrix_memory_recurrence: bad decay row stride");
     if (num_seqs <= 0) return VMX_OK;
-    const DeltaArgs a{q, k, v, g, beta, ldq, ldk, ldv, ldg, ldbeta, o, ldo, state, positions, seq_starts, state_slots, heads, qk_heads, dim, vdim,
-                      g_per_head ? 1 : 0, beta ? 0 : 1, q_mul};
-    const dim3 grid((vdim + DR_VT - 1) / DR_VT, heads, num_seqs);
+    const bool gain = opts && opts->write_gain, norm = opts && opts->norm_out;
+    VMX_REQUIRE(!(gain && beta), "matrix_memory_recurrence: a write gain belongs to the plain write, beta to the delta rule");
+    VMX_REQUIRE(!norm || opts->ldnorm >= heads, "matrix_memory_recurrence: bad row stride of the normaliser's read-out");
+    const DeltaArgs a{q, k, v, g, gain ? opts->write_gain : beta, ldq, ldk, ldv, ldg, gain ? opts->ldgain : ldbeta, o, ldo, state, positions,
+                      seq_starts, state_slots, heads, qk_heads, dim, vdim, g_per_head ? 1 : 0, beta ? 0 : 1, q_mul, norm ? opts->norm_out : nullptr,
+                      norm ? opts->ldnorm : 0};
+    const dim3 grid((vdim + (norm ? 1 : 0) + DR_VT - 1) / DR_VT, heads, num_seqs);
     hipStream_t st = vmx_stream(stream);
     int rc;
     switch (delta_dpt(dim)) {
@@ -405,12 +474,32 @@ extern "C" int vmx_head_rms_gate(void *y, int y_dtype, const float *o, int64_t l
 }
 
 extern "C" int vmx_head_rms_gate_ex(void *y, int y_dtype, const float *o, int64_t ldo, const uint16_t *w_bf16, const float *gate, int64_t ldgate,
-                                    int gate_silu, float eps, int tokens, int heads, int vdim, void *stream) {
-    VMX_REQUIRE(y && o, "head_rms_gate: null pointer");
+                                       int gate_silu, float eps, int tokens, int heads, int vdim, void *stream) {
+    const vmx_read_out_opts ro = {gate_silu, 0, nullptr, 0, nullptr, 0, 0.f};
+    return vmx_head_read_out(y, y_dtype, o, ldo, w_bf16, gate, ldgate, eps, tokens, heads, vdim, &ro, stream);
+}
+
+extern "C" int vmx_exp_gate_scan(float *input_gate, int64_t ldi, float *forget_gate, int64_t ldf, float *floor, int64_t ldfloor, float *max_state,
+                                 float cap, const int32_t *positions, const int32_t *seq_starts, const int32_t *state_slots, int num_seqs,
+                                 int heads, void *stream) {
+    VMX_REQUIRE(input_gate && forget_gate && floor && max_state && positions && seq_starts && state_slots, "exp_gate_scan: null pointer");
+    VMX_REQUIRE(heads >= 1 && ldi >= heads && ldf >= heads && ldfloor >= heads && cap > 0.f, "exp_gate_scan: bad sizes or cap");
+    if (num_seqs <= 0) return VMX_OK;
+    hipLaunchKernelGGL(exp_gate_scan_kernel, dim3(heads, num_seqs), dim3(64), 0, vmx_stream(stream), input_gate, ldi, forget_gate, ldf, floor, ldfloor,
+                       max_state, cap, positions, seq_starts, state_slots, heads);
+    VMX_CHECK_LAUNCH("exp_gate_scan");
+    return VMX_OK;
+}
+
+extern "C" int vmx_head_read_out(void *y, int y_dtype, const float *o, int64_t ldo, const uint16_t *w_bf16, const float *gate, int64_t ldgate,
+                                 float eps, int tokens, int heads, int vdim, const vmx_read_out_opts *opts, void *stream) {
+    VMX_REQUIRE(y && o && opts, "head_rms_gate: null pointer");
+    VMX_REQUIRE(!opts->norm || opts->floor, "head_rms_gate: a normaliser comes with its floor");
     VMX_REQUIRE(y_dtype == VMX_F32 || y_dtype == VMX_BF16, "head_rms_gate: f32 or bf16 output");
     if (tokens <= 0) return VMX_OK;
     hipLaunchKernelGGL(head_rms_gate_kernel, dim3((tokens * heads + 3) / 4), dim3(256), 0, vmx_stream(stream), y, y_dtype == VMX_F32, o, ldo,
-                       w_bf16, gate, ldgate, eps, tokens * heads, heads, vdim, gate_silu ? 1 : 0);
+                       w_bf16, gate, ldgate, eps, tokens * heads, heads, vdim, opts->gate_silu ? 1 : 0, opts->w_per_head ? 1 : 0, opts->norm,
+                       opts->ldnorm, opts->floor, opts->ldfloor, opts->norm_eps);
     VMX_CHECK_LAUNCH("head_rms_gate");
     return VMX_OK;
 }

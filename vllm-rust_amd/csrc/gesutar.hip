@@ -63,16 +63,6 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(float *__restrict__ x
     }
 }
 
-// out[h][r][d] = in[h][d][r]: the key up-projection as [head][latent][dim], so that qa_h = U_h^T q_h reads its weights along k
-__global__ __launch_bounds__(256) void transpose_heads_kernel(uint16_t *__restrict__ out, const uint16_t *__restrict__ in, int H, int D, int R) {
-    const int64_t n = (int64_t)H * D * R;
-    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
-        const int64_t h = i / ((int64_t)D * R), rem = i % ((int64_t)D * R);
-        const int r = (int)(rem / D), d = (int)(rem % D);
-        out[i] = in[(h * D + d) * R + r];
-    }
-}
-
 int upload(Buf &b, size_t offset, const void *data, size_t bytes, hipStream_t st) {
     VMX_CHECK_HIP(hipMemcpyAsync((char *)b.p + offset, data, bytes, hipMemcpyDefault, st));
     VMX_CHECK_HIP(hipStreamSynchronize(st));
@@ -306,9 +296,7 @@ extern "C" int vmx_gesutar_load_tensor(vmx_gesutar *m, const char *name, const v
         if (int rc = upload(*dst, off, data, bytes, st)) return rc;
         if (n.size() > 7 && n.compare(n.size() - 7, 7, ".mix.uk") == 0) {
             Layer &L = m->layers[atoi(n.substr(1).c_str())];
-            hipLaunchKernelGGL(transpose_heads_kernel, dim3(512), dim3(256), 0, st, L.uk_t.as<uint16_t>(), L.uk.as<uint16_t>(), L.c.heads, L.c.dim,
-                               L.c.kv_rank);
-            VMX_CHECK_LAUNCH("gesutar transpose");
+            if (int rc = vmx_latent_transpose_heads(L.uk_t.as<uint16_t>(), L.uk.as<uint16_t>(), L.c.heads, L.c.dim, L.c.kv_rank, st)) return rc;
             VMX_CHECK_HIP(hipStreamSynchronize(st));
         }
     }

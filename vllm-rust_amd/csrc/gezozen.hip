@@ -113,31 +113,6 @@ int upload_rotation(const vmx_rotation &r, Buf &steps, float &mul) {
 
 }  // namespace
 
-extern "C" int vmx_rotation_steps(const vmx_rotation *rot, float *steps, float *mul) {
-    VMX_REQUIRE(rot && steps && mul, "rotation_steps: null pointer");
-    const vmx_rotation &r = *rot;
-    VMX_REQUIRE(r.dims >= 2 && r.dims % 2 == 0 && r.base > 1.0, "rotation_steps: %d rotated coordinates, base %g", r.dims, r.base);
-    const int half = r.dims / 2;
-    *mul = 1.f;
-    double lo = 0, hi = 0;
-    if (r.factor > 0.0) {
-        VMX_REQUIRE(r.original > 0.0 && r.fast > 0.0 && r.slow > 0.0, "rotation_steps: bad stretch constants");
-        auto idx = [&](double turns) { return r.dims * log(r.original / (2.0 * M_PI * turns)) / (2.0 * log(r.base)); };
-        lo = std::max(floor(idx(r.fast)), 0.0);
-        hi = std::min(ceil(idx(r.slow)), (double)(r.dims - 1));
-        *mul = (float)(0.1 * log(r.factor) + 1.0);
-    }
-    for (int i = 0; i < half; i++) {
-        double f = pow(r.base, -2.0 * i / r.dims);
-        if (r.factor > 0.0) {
-            const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
-            f = f / r.factor * ramp + f * (1.0 - ramp);
-        }
-        steps[i] = (float)f;
-    }
-    return VMX_OK;
-}
-
 extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezozen_layer_config *layer_cfgs, vmx_gezozen **out) {
     VMX_REQUIRE(cfg && layer_cfgs && out, "gezozen_create: null pointer");
     const vmx_gezozen_config &c = *cfg;

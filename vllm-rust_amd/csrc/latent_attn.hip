@@ -8,7 +8,9 @@
 //
 // Parameters rather than constants: window (position i sees j with 0 <= i - j < window; 0 = unbounded causal), an optional
 // per-head sink logit (a key-less term exp(sink_h) in the softmax denominator, not scaled), the rotation (interleaved pairs
-// (2i, 2i+1) of the first rot_dims dimensions, angle = position * inv_freq[i]), sizes, cache element type (bf16 / f32).
+// (2i, 2i+1) or halves (i, i + rot_dims / 2) of the first rot_dims dimensions, angle = position * inv_freq[i], cos and sin times a
+// constant), queries straight from the input or through an RMS-normed latent of their own, sizes, cache element type (bf16 / f32).
+// Layers may attend over another layer's cache: preparation then skips the key/value part.
 // Scores, softmax, the weighted sum, norms and angles are f32.  Queries are packed: token t belongs to sequence seq_ids[t] at
 // position positions[t], so prompts of different lengths, prompt portions and single decode tokens are the same launch, and a
 // token's result depends only on its own query and the cache rows of its window.
@@ -26,59 +28,85 @@ template <bool F32> __device__ __forceinline__ void st_cache(void *c, int64_t i,
     else ((uint16_t *)c)[i] = vmx_f32_to_bf16(v);
 }
 
-// One workgroup per token: c = rms_norm(dkv[:R]) * w, k_rot = rotate(dkv[R:]) -> cache row `slot`; rotate(q_h[dim:]) -> q_rot.
-template <bool F32>
-__global__ __launch_bounds__(256) void latent_prepare_kernel(const float *__restrict__ fused, int64_t ldf, int q_off, int dkv_off,
-                                                              const uint16_t *__restrict__ norm_w, float eps,
-                                                              const float *__restrict__ inv_freq, int rot_dims,
-                                                              const int32_t *__restrict__ positions, const int32_t *__restrict__ slots,
-                                                              void *__restrict__ cache, float *__restrict__ q_rot, int H, int dim, int rd,
-                                                              int R) {
+struct LatentPrepareArgs {
+    vmx_latent_prepare p;
+    const int32_t *positions, *slots;
+    void *cache, *q_latent_out;
+};
+
+// One workgroup per token, any of three parts (a part without its input pointer is skipped):
+//   q_latent: RMS-normed row of the query's latent -> q_latent_out (the element type of the cache);
+//   kv:       c = rms_norm(kv[:R]) * w, k_rot = rotate(kv[R:]) -> cache row `slot`;
+//   q:        rotate(q_h[dim:]) -> q_rot.
+template <bool F32> __global__ __launch_bounds__(256) void latent_prepare_kernel(const LatentPrepareArgs a) {
     __shared__ float red[4];
+    __shared__ float2 turn[128];     // cos and sin of the token's angles, shared by all heads
+    const vmx_latent_prepare &p = a.p;
     const int t = blockIdx.x, tid = threadIdx.x;
-    const float *row = fused + (int64_t)t * ldf;
-    const float pos = (float)positions[t];
-    const int64_t slot = slots[t];
-    float ss = 0.f;
-    for (int i = tid; i < R; i += 256) {
-        const float v = row[dkv_off + i];
-        ss += v * v;
+    const float pos = (float)a.positions[t];
+    if (p.q_latent) {
+        const float *row = p.q_latent + (int64_t)t * p.ldq_latent;
+        float ss = 0.f;
+        for (int i = tid; i < p.q_rank; i += 256) ss = fmaf(row[i], row[i], ss);
+        ss = vmx_block_sum_256(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)p.q_rank + p.eps);
+        for (int i = tid; i < p.q_rank; i += 256)
+            st_cache<F32>(a.q_latent_out, (int64_t)t * p.q_rank + i, row[i] * inv * vmx_bf16_to_f32(p.q_latent_norm_bf16[i]));
     }
-    ss = vmx_block_sum_256(ss, red);
-    const float inv = 1.0f / sqrtf(ss / (float)R + eps);
-    void *crow = cache;
+    const int R = p.kv_rank, rd = p.rot_dim, half = p.rot_dims >> 1, nq = p.q ? p.heads : 0;
+    const float *kv = p.kv ? p.kv + (int64_t)t * p.ldkv : nullptr;
+    const int64_t slot = kv ? a.slots[t] : -1;
     const int64_t cbase = slot * (R + rd);
-    if (slot >= 0) {
-        for (int i = tid; i < R; i += 256) st_cache<F32>(crow, cbase + i, row[dkv_off + i] * inv * vmx_bf16_to_f32(norm_w[i]));
+    if (kv) {
+        float ss = 0.f;
+        for (int i = tid; i < R; i += 256) ss += kv[i] * kv[i];
+        ss = vmx_block_sum_256(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)R + p.eps);
+        if (slot >= 0)
+            for (int i = tid; i < R; i += 256) st_cache<F32>(a.cache, cbase + i, kv[i] * inv * vmx_bf16_to_f32(p.latent_norm_bf16[i]));
     }
-    // rotations: work item = (vector v, pair i); vector 0 is the shared key part, vector 1 + h the rotated part of head h's query
-    const int half = rot_dims >> 1;
-    for (int w = tid; w < (H + 1) * half; w += 256) {
-        const int v = w / half, i = w % half;
+    if (!kv && !nq) return;
+    auto angle = [&](int i) {
         float sn, cs;
-        sincosf(pos * inv_freq[i], &sn, &cs);
-        const float *src = v == 0 ? row + dkv_off + R : row + q_off + (int64_t)(v - 1) * (dim + rd) + dim;
-        const float a = src[2 * i], b = src[2 * i + 1];
-        const float ra = a * cs - b * sn, rb = b * cs + a * sn;
+        sincosf(pos * p.inv_freq[i], &sn, &cs);
+        return make_float2(cs * p.rot_mul, sn * p.rot_mul);
+    };
+    for (int i = tid; i < min(half, 128); i += 256) turn[i] = angle(i);
+    __syncthreads();
+    // rotations: work item = (vector v, pair i); vector 0 is the shared key part, vector 1 + h the rotated part of head h's query
+    const int v0 = slot >= 0 ? 0 : 1;
+    for (int w = tid + v0 * half; w < (nq + 1) * half; w += 256) {
+        const int v = w / half, i = w % half;
+        const float2 cs = i < 128 ? turn[i] : angle(i);
+        const float *src = v == 0 ? kv + R : p.q + (int64_t)t * p.ldq + (int64_t)(v - 1) * (p.dim + rd) + p.dim;
+        const int ia = p.rot_halves ? i : 2 * i, ib = p.rot_halves ? i + half : 2 * i + 1;
+        const float x = src[ia], y = src[ib];
+        const float rx = x * cs.x - y * cs.y, ry = y * cs.x + x * cs.y;
         if (v == 0) {
-            if (slot >= 0) {
-                st_cache<F32>(crow, cbase + R + 2 * i, ra);
-                st_cache<F32>(crow, cbase + R + 2 * i + 1, rb);
-            }
+            st_cache<F32>(a.cache, cbase + R + ia, rx);
+            st_cache<F32>(a.cache, cbase + R + ib, ry);
         } else {
-            float *dst = q_rot + ((int64_t)t * H + (v - 1)) * rd;
-            dst[2 * i] = ra;
-            dst[2 * i + 1] = rb;
+            float *dst = p.q_rot + ((int64_t)t * nq + (v - 1)) * rd;
+            dst[ia] = rx;
+            dst[ib] = ry;
         }
     }
     // dimensions past rot_dims pass unchanged
-    for (int w = tid; w < (H + 1) * (rd - rot_dims); w += 256) {
-        const int v = w / (rd - rot_dims), i = rot_dims + w % (rd - rot_dims);
-        if (v == 0) {
-            if (slot >= 0) st_cache<F32>(crow, cbase + R + i, row[dkv_off + R + i]);
-        } else {
-            q_rot[((int64_t)t * H + (v - 1)) * rd + i] = row[q_off + (int64_t)(v - 1) * (dim + rd) + dim + i];
-        }
+    const int rest = rd - p.rot_dims;
+    for (int w = tid + v0 * rest; w < (nq + 1) * rest; w += 256) {
+        const int v = w / rest, i = p.rot_dims + w % rest;
+        if (v == 0) st_cache<F32>(a.cache, cbase + R + i, kv[R + i]);
+        else p.q_rot[((int64_t)t * nq + (v - 1)) * rd + i] = p.q[(int64_t)t * p.ldq + (int64_t)(v - 1) * (p.dim + rd) + p.dim + i];
+    }
+}
+
+// out[h][r][d] = in[h][d][r]: the key up-projection as [head][latent][dim], so that qa_h = U_h^T q_h reads its weights along k
+__global__ __launch_bounds__(256) void transpose_heads_kernel(uint16_t *__restrict__ out, const uint16_t *__restrict__ in, int H, int D, int R) {
+    const int64_t n = (int64_t)H * D * R;
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+        const int64_t h = i / ((int64_t)D * R), rem = i % ((int64_t)D * R);
+        const int r = (int)(rem / D), d = (int)(rem % D);
+        out[i] = in[(h * D + d) * R + r];
     }
 }
 
@@ -421,23 +449,41 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(float *__restric
 
 }  // namespace
 
+extern "C" int vmx_latent_prepare_rows(const vmx_latent_prepare *prep, const int32_t *positions, const int32_t *slots, void *cache,
+                                       int cache_dtype, void *q_latent_out, int tokens, void *stream) {
+    VMX_REQUIRE(prep && positions, "latent_prepare: null pointer");
+    const vmx_latent_prepare &p = *prep;
+    VMX_REQUIRE(cache_dtype == VMX_F32 || cache_dtype == VMX_BF16, "latent_prepare: the cache holds f32 or bf16");
+    VMX_REQUIRE(!p.kv || (slots && cache && p.latent_norm_bf16 && p.kv_rank >= 1 && p.ldkv >= p.kv_rank + p.rot_dim), "latent_prepare: bad key/value rows");
+    VMX_REQUIRE(!p.q || (p.heads >= 1 && p.dim >= 0 && p.rot_dim >= 0 && p.ldq >= (int64_t)p.heads * (p.dim + p.rot_dim) && (p.q_rot || p.rot_dim == 0)),
+                "latent_prepare: bad query rows");
+    VMX_REQUIRE(!p.q_latent || (q_latent_out && p.q_latent_norm_bf16 && p.q_rank >= 1 && p.ldq_latent >= p.q_rank), "latent_prepare: bad query latents");
+    VMX_REQUIRE(!(p.kv || p.q) || (p.rot_dims >= 0 && p.rot_dims <= p.rot_dim && p.rot_dims % 2 == 0 && (p.inv_freq || p.rot_dims == 0)),
+                "latent_prepare: rot_dims (%d) must be even and at most rot_dim (%d)", p.rot_dims, p.rot_dim);
+    if (tokens <= 0) return VMX_OK;
+    LatentPrepareArgs a{p, positions, slots, cache, q_latent_out};
+    if (a.p.rot_mul == 0.f) a.p.rot_mul = 1.f;
+    if (cache_dtype == VMX_F32) hipLaunchKernelGGL(latent_prepare_kernel<true>, dim3(tokens), dim3(256), 0, vmx_stream(stream), a);
+    else hipLaunchKernelGGL(latent_prepare_kernel<false>, dim3(tokens), dim3(256), 0, vmx_stream(stream), a);
+    VMX_CHECK_LAUNCH("latent_prepare");
+    return VMX_OK;
+}
+
 extern "C" int vmx_latent_kv_prepare(const float *fused, int64_t ld_fused, int q_offset, int dkv_offset, const uint16_t *latent_norm_w,
                                      float eps, const float *inv_freq, int rot_dims, const int32_t *positions, const int32_t *slots,
                                      void *cache, int cache_dtype, float *q_rot, int tokens, int heads, int dim, int rot_dim, int kv_rank,
                                      void *stream) {
     VMX_REQUIRE(fused && latent_norm_w && inv_freq && positions && slots && cache && q_rot, "latent_kv_prepare: null pointer");
-    VMX_REQUIRE(cache_dtype == VMX_F32 || cache_dtype == VMX_BF16, "latent_kv_prepare: the cache holds f32 or bf16");
-    VMX_REQUIRE(heads >= 1 && dim >= 0 && rot_dim >= 0 && kv_rank >= 1, "latent_kv_prepare: bad sizes");
-    VMX_REQUIRE(rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0, "latent_kv_prepare: rot_dims (%d) must be even and at most rot_dim (%d)",
-                rot_dims, rot_dim);
-    if (tokens <= 0) return VMX_OK;
-    if (cache_dtype == VMX_F32)
-        hipLaunchKernelGGL(latent_prepare_kernel<true>, dim3(tokens), dim3(256), 0, vmx_stream(stream), fused, ld_fused, q_offset, dkv_offset,
-                           latent_norm_w, eps, inv_freq, rot_dims, positions, slots, cache, q_rot, heads, dim, rot_dim, kv_rank);
-    else
-        hipLaunchKernelGGL(latent_prepare_kernel<false>, dim3(tokens), dim3(256), 0, vmx_stream(stream), fused, ld_fused, q_offset, dkv_offset,
-                           latent_norm_w, eps, inv_freq, rot_dims, positions, slots, cache, q_rot, heads, dim, rot_dim, kv_rank);
-    VMX_CHECK_LAUNCH("latent_kv_prepare");
+    vmx_latent_prepare p = {};
+    p.kv = fused + dkv_offset, p.ldkv = ld_fused, p.kv_rank = kv_rank, p.latent_norm_bf16 = latent_norm_w, p.eps = eps;
+    p.q = fused + q_offset, p.ldq = ld_fused, p.heads = heads, p.dim = dim, p.rot_dim = rot_dim, p.q_rot = q_rot;
+    p.inv_freq = inv_freq, p.rot_dims = rot_dims, p.rot_mul = 1.0f;
+    return vmx_latent_prepare_rows(&p, positions, slots, cache, cache_dtype, nullptr, tokens, stream);
+}
+
+int vmx_latent_transpose_heads(uint16_t *out, const uint16_t *in, int heads, int dim, int kv_rank, hipStream_t st) {
+    hipLaunchKernelGGL(transpose_heads_kernel, dim3(512), dim3(256), 0, st, out, in, heads, dim, kv_rank);
+    VMX_CHECK_LAUNCH("latent transpose");
     return VMX_OK;
 }
 

@@ -2,7 +2,8 @@
 // group-limited choice) and the token -> expert alignment that sorts (token, slot) pairs into expert blocks.
 // Semantics: crates/core/kernels/topk_softmax.cu:63-311 (softmax with expf, max-subtracted; k rounds of argmax, ties -> smaller
 // index; optional renormalisation by the selected sum) and crates/core/kernels/fused_moe_align.cu:34-278 (moe_align_block_size).
-// Sigmoid scores (vmx_topk_sigmoid): every expert's logit goes through the logistic function by itself; same selection.
+// Sigmoid scores (vmx_topk_sigmoid): every expert's logit goes through the logistic function by itself; same selection.  Group-limited
+// choice over softmax scores (vmx_grouped_topk_router) or over corrected sigmoid scores (vmx_grouped_topk_sigmoid).
 #include "vmx_kernels.h"
 #include <float.h>
 
@@ -89,13 +90,18 @@ __device__ __forceinline__ void wave_argmax(float &bv, int &bi) {
     argmax_step<1>(bv, bi);
 }
 
-// Router with group-limited selection: softmax over all experts; the experts form `groups` equal runs of neighbours, a group's
-// score is its largest probability, and only experts of the `keep` best groups can be chosen; then k rounds of argmax (ties ->
-// smaller index) over what is left.  Weights: the chosen probabilities divided by (their sum + 1e-20), times `scale`.
-// One wave per token; lane l holds experts (and groups) l, l + 64, ...: E <= 256.
-__global__ __launch_bounds__(256) void grouped_topk_router_kernel(const float *__restrict__ logits, float *__restrict__ w_out,
-                                                                   int32_t *__restrict__ id_out, int tokens, int E, int k, int groups,
-                                                                   int keep, float scale) {
+// Router with group-limited selection; the experts form `groups` equal runs of neighbours, only experts of the `keep` best groups
+// can be chosen; then k rounds of argmax (ties -> smaller index) over what is left.  Two scorings:
+//   SIGMOID = false: softmax over all experts, a group's score is its largest probability; weights: the chosen probabilities
+//                    divided by (their sum + 1e-20), times `scale`;
+//   SIGMOID = true:  every expert's logit through the logistic function; the CHOICE is made on score + correction (which may be
+//                    negative), a group's score is the sum of its two largest choice scores; weights: the chosen scores without
+//                    the correction, times `scale`, not renormalised.
+// One wave per token; lane l holds experts (and groups) l, l + 64, ...: E <= 256.  Logits rows are ld numbers apart.
+template <bool SIGMOID>
+__global__ __launch_bounds__(256) void grouped_topk_router_kernel(const float *__restrict__ logits, int64_t ld, const uint16_t *__restrict__ correction,
+                                                                   float *__restrict__ w_out, int32_t *__restrict__ id_out, int tokens, int E, int k,
+                                                                   int groups, int keep, float scale) {
     __shared__ float sc[4][256];
     __shared__ int32_t ok[4][256];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = blockIdx.x * 4 + wave;
@@ -105,19 +111,29 @@ __global__ __launch_bounds__(256) void grouped_topk_router_kernel(const float *_
 #pragma unroll
     for (int j = 0; j < 4; j++) {
         const int e = lane + 64 * j;
-        v[j] = e < E ? logits[(int64_t)t * E + e] : -FLT_MAX;
+        v[j] = e < E ? logits[(int64_t)t * ld + e] : -FLT_MAX;
         mx = fmaxf(mx, v[j]);
     }
-    mx = vmx_wave_max(mx);
-    float sum = 0.f;
+    float s[4];   // SIGMOID: the scores without the correction (v: the choice scores)
+    if constexpr (SIGMOID) {
 #pragma unroll
-    for (int j = 0; j < 4; j++) {
-        v[j] = (lane + 64 * j < E) ? expf(v[j] - mx) : 0.f;
-        sum += v[j];
+        for (int j = 0; j < 4; j++) {
+            const int e = lane + 64 * j;
+            s[j] = 1.0f / (1.0f + expf(-v[j]));
+            v[j] = e < E ? s[j] + vmx_bf16_to_f32(correction[e]) : -FLT_MAX;
+        }
+    } else {
+        mx = vmx_wave_max(mx);
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            v[j] = (lane + 64 * j < E) ? expf(v[j] - mx) : 0.f;
+            sum += v[j];
+        }
+        sum = vmx_wave_sum(sum);
+#pragma unroll
+        for (int j = 0; j < 4; j++) v[j] = (lane + 64 * j < E) ? v[j] / sum : -FLT_MAX;
     }
-    sum = vmx_wave_sum(sum);
-#pragma unroll
-    for (int j = 0; j < 4; j++) v[j] = (lane + 64 * j < E) ? v[j] / sum : -FLT_MAX;
     if (groups > 1 && keep < groups) {
         const int gs = E / groups;
 #pragma unroll
@@ -128,8 +144,15 @@ __global__ __launch_bounds__(256) void grouped_topk_router_kernel(const float *_
         for (int j = 0; j < 4; j++) {
             const int g = lane + 64 * j;
             gv[j] = -FLT_MAX;
-            if (g < groups)
-                for (int i = 0; i < gs; i++) gv[j] = fmaxf(gv[j], sc[wave][g * gs + i]);
+            if (g < groups) {
+                float second = -FLT_MAX;
+                for (int i = 0; i < gs; i++) {
+                    const float x = sc[wave][g * gs + i];
+                    second = fmaxf(second, fminf(x, gv[j]));
+                    gv[j] = fmaxf(gv[j], x);
+                }
+                if (SIGMOID && gs > 1) gv[j] += second;
+            }
             ok[wave][g] = 0;
         }
         __builtin_amdgcn_wave_barrier();
@@ -163,13 +186,20 @@ __global__ __launch_bounds__(256) void grouped_topk_router_kernel(const float *_
             if (e < E && v[j] > bv) { bv = v[j]; bi = e; }
         }
         wave_argmax(bv, bi);
-        if (lane == 0) { w_out[(int64_t)t * k + ki] = bv; id_out[(int64_t)t * k + ki] = bi; }
-        selected += bv;
+        if (bi >= E) bi = 0;   // only when every logit left is not a number
+        if constexpr (SIGMOID) {
+#pragma unroll
+            for (int j = 0; j < 4; j++)
+                if (lane + 64 * j == bi) { w_out[(int64_t)t * k + ki] = s[j] * scale; id_out[(int64_t)t * k + ki] = bi; }
+        } else {
+            if (lane == 0) { w_out[(int64_t)t * k + ki] = bv; id_out[(int64_t)t * k + ki] = bi; }
+            selected += bv;
+        }
 #pragma unroll
         for (int j = 0; j < 4; j++)
             if (lane + 64 * j == bi) v[j] = -FLT_MAX;
     }
-    if (lane == 0) {
+    if (!SIGMOID && lane == 0) {
         const float f = scale / (selected + 1e-20f);
         for (int ki = 0; ki < k; ki++) w_out[(int64_t)t * k + ki] *= f;
     }
@@ -323,18 +353,35 @@ static int topk_scores(const void *logits, int logits_dtype, float *topk_weights
     return VMX_OK;
 }
 
-extern "C" int vmx_grouped_topk_router(const float *logits, float *topk_weights, int32_t *topk_ids, int tokens, int num_experts, int k,
-                                       int groups, int keep_groups, float scale, void *stream) {
+static int grouped_router(const float *logits, int64_t ld, const uint16_t *correction, float *topk_weights, int32_t *topk_ids, int tokens,
+                          int num_experts, int k, int groups, int keep_groups, float scale, void *stream) {
     VMX_REQUIRE(logits && topk_weights && topk_ids, "grouped_topk_router: null pointer");
-    VMX_REQUIRE(num_experts >= 1 && num_experts <= 256, "grouped_topk_router: num_experts (%d) must be in 1..256", num_experts);
+    VMX_REQUIRE(num_experts >= 1 && num_experts <= 256 && ld >= num_experts, "grouped_topk_router: num_experts (%d) must be in 1..256", num_experts);
     VMX_REQUIRE(groups >= 1 && num_experts % groups == 0, "grouped_topk_router: %d experts do not form %d equal groups", num_experts, groups);
     VMX_REQUIRE(keep_groups >= 1 && keep_groups <= groups, "grouped_topk_router: keep_groups (%d) must be in 1..groups", keep_groups);
     VMX_REQUIRE(k >= 1 && k <= keep_groups * (num_experts / groups), "grouped_topk_router: k (%d) exceeds the experts of the kept groups", k);
     if (tokens <= 0) return VMX_OK;
-    hipLaunchKernelGGL(grouped_topk_router_kernel, dim3((tokens + 3) / 4), dim3(256), 0, vmx_stream(stream), logits, topk_weights, topk_ids,
-                       tokens, num_experts, k, groups, keep_groups, scale);
+    const dim3 grid((tokens + 3) / 4), block(256);
+    if (correction)
+        hipLaunchKernelGGL(grouped_topk_router_kernel<true>, grid, block, 0, vmx_stream(stream), logits, ld, correction, topk_weights, topk_ids, tokens,
+                           num_experts, k, groups, keep_groups, scale);
+    else
+        hipLaunchKernelGGL(grouped_topk_router_kernel<false>, grid, block, 0, vmx_stream(stream), logits, ld, correction, topk_weights, topk_ids, tokens,
+                           num_experts, k, groups, keep_groups, scale);
     VMX_CHECK_LAUNCH("grouped_topk_router");
     return VMX_OK;
+}
+
+extern "C" int vmx_grouped_topk_router(const float *logits, float *topk_weights, int32_t *topk_ids, int tokens, int num_experts, int k,
+                                       int groups, int keep_groups, float scale, void *stream) {
+    return grouped_router(logits, num_experts, nullptr, topk_weights, topk_ids, tokens, num_experts, k, groups, keep_groups, scale, stream);
+}
+
+extern "C" int vmx_grouped_topk_sigmoid(const float *logits, int64_t ld_logits, const uint16_t *correction_bf16, float *topk_weights,
+                                        int32_t *topk_ids, int tokens, int num_experts, int k, int groups, int keep_groups, float scale,
+                                        void *stream) {
+    VMX_REQUIRE(correction_bf16, "grouped_topk_sigmoid: null pointer");
+    return grouped_router(logits, ld_logits, correction_bf16, topk_weights, topk_ids, tokens, num_experts, k, groups, keep_groups, scale, stream);
 }
 
 extern "C" int vmx_moe_align_block_size(const int32_t *topk_ids, int32_t *sorted_token_ids, int32_t *expert_ids,

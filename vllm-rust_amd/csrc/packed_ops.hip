@@ -1,15 +1,20 @@
-// Kernels that every packed-step executor needs around its mixers and linears: RMS norm of the f32 residual stream (a gain per
-// column or one gain for the row), the inverse map and the weighted combine of a mixture of experts whose (token, slot) pairs were
-// sorted into expert blocks, greedy ids of f32 logits rows, a fill.
+// Kernels that every packed-step executor needs around its mixers and linears: RMS and layer norm of the f32 residual stream (a
+// gain per column or one gain for the row), the norms on both sides of a residual sum in one pass, gated activations, the inverse
+// map and the weighted combine of a mixture of experts whose (token, slot) pairs were sorted into expert blocks, greedy ids of f32
+// logits rows, a fill, the step table of a rotary position code.
 #include "vmx_kernels.h"
 #include <float.h>
+#include <math.h>
+#include <algorithm>
 
 namespace {
 
 // out[r] = x[rows ? rows[r] : r] / sqrt(mean(x^2) + eps) * w, f32 statistics; out in f32 or bf16; w one gain per column or
-// (w_scalar) a single gain for the whole row.  Rows up to 4096 wide stay
-// in registers between the statistic and the scaling (one trip to memory), wider rows are read twice.
-__global__ __launch_bounds__(256) void rms_norm_f32in_kernel(void *__restrict__ out, int out_f32, const float *__restrict__ x,
+// (w_scalar) a single gain for the whole row.  CENTERED: the row's mean is taken off first (layer norm; the statistic is then the
+// variance).  Rows up to 4096 wide stay in registers between the statistics and the scaling (one trip to memory), wider rows are
+// read once per pass.
+template <bool CENTERED>
+__global__ __launch_bounds__(256) void row_norm_f32in_kernel(void *__restrict__ out, int out_f32, const float *__restrict__ x,
                                                               const int32_t *__restrict__ rows, const uint16_t *__restrict__ w, int w_scalar,
                                                               int width, float eps) {
     __shared__ float red[4];
@@ -18,7 +23,7 @@ __global__ __launch_bounds__(256) void rms_norm_f32in_kernel(void *__restrict__ 
     constexpr int PT = 16;
     float xv[PT], wv[PT];
     const bool held = width <= 256 * PT;
-    float ss = 0.f;
+    float ss = 0.f, mean = 0.f;
     if (held) {
 #pragma unroll
         for (int u = 0; u < PT; u++) {
@@ -26,10 +31,23 @@ __global__ __launch_bounds__(256) void rms_norm_f32in_kernel(void *__restrict__ 
             xv[u] = i < width ? src[i] : 0.f;
             wv[u] = i < width ? vmx_bf16_to_f32(w[w_scalar ? 0 : i]) : 0.f;
         }
+        if constexpr (CENTERED) {
+            float s = 0.f;
+#pragma unroll
+            for (int u = 0; u < PT; u++) s += xv[u];
+            mean = vmx_block_sum_256(s, red) / (float)width;
+#pragma unroll
+            for (int u = 0; u < PT; u++) xv[u] = threadIdx.x + 256 * u < width ? xv[u] - mean : 0.f;
+        }
 #pragma unroll
         for (int u = 0; u < PT; u++) ss += xv[u] * xv[u];   // same order as the strided loop below
     } else {
-        for (int i = threadIdx.x; i < width; i += 256) ss += src[i] * src[i];
+        if constexpr (CENTERED) {
+            float s = 0.f;
+            for (int i = threadIdx.x; i < width; i += 256) s += src[i];
+            mean = vmx_block_sum_256(s, red) / (float)width;
+        }
+        for (int i = threadIdx.x; i < width; i += 256) ss += (src[i] - mean) * (src[i] - mean);
     }
     ss = vmx_block_sum_256(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)width + eps);
@@ -46,9 +64,96 @@ __global__ __launch_bounds__(256) void rms_norm_f32in_kernel(void *__restrict__ 
         return;
     }
     for (int i = threadIdx.x; i < width; i += 256) {
-        const float v = src[i] * inv * vmx_bf16_to_f32(w[w_scalar ? 0 : i]);
+        const float v = (src[i] - mean) * inv * vmx_bf16_to_f32(w[w_scalar ? 0 : i]);
         if (out_f32) ((float *)out)[(int64_t)r * width + i] = v;
         else ((uint16_t *)out)[(int64_t)r * width + i] = vmx_f32_to_bf16(v);
+    }
+}
+
+// Both norms around a residual sum in one pass over the row: x <- [x +] N(y) * w_post, h = N(x) * w_next (w_next NULL: no h).
+// y[t] is a row of numbers, a row of the embedding table, or the combined result of a mixture of experts.  N as above, centred or
+// not.  HELD > 0: a thread keeps its HELD numbers of the row in registers from the first read to the last store; 0: any width, y
+// is formed anew in every pass (at most three) and the new x is read back by the thread that wrote it.
+template <int HELD>
+__global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a) {
+    __shared__ float red[4];
+    constexpr int PT = HELD ? HELD : 1;
+    const int t = blockIdx.x, W = a.width;
+    float *x = a.x + (int64_t)t * W;
+    const float inv_w = 1.0f / (float)W;
+    int64_t erow = 0;
+    if (a.embed) {
+        const int id = a.tokens[t];
+        erow = (int64_t)(id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id)) * W;
+    }
+    const float sg = a.shared_gate ? 1.0f / (1.0f + expf(-a.shared_gate[(int64_t)t * a.ld_shared_gate])) : 1.0f;
+    auto y_at = [&](int i) {
+        if (a.embed) return vmx_bf16_to_f32(a.embed[erow + i]);
+        if (!a.pair_rows) return a.y[(int64_t)t * W + i];
+        float v = 0.f;
+        for (int s = 0; s < a.top; s++) v = fmaf(a.pair_w[(int64_t)t * a.top + s], a.y[(int64_t)a.pair_rows[(int64_t)t * a.top + s] * W + i], v);
+        if (a.shared) v = fmaf(sg, a.shared[(int64_t)t * W + i], v);
+        return v;
+    };
+    // sum of f over the row's columns, in the same order for every HELD
+    float held[PT];
+    auto over_row = [&](auto &&f) {
+        float s = 0.f;
+        if constexpr (HELD > 0) {
+#pragma unroll
+            for (int u = 0; u < PT; u++)
+                if (threadIdx.x + 256 * u < W) s += f(threadIdx.x + 256 * u, u);
+        } else {
+            for (int i = threadIdx.x; i < W; i += 256) s += f(i, 0);
+        }
+        return vmx_block_sum_256(s, red);
+    };
+    auto norm_of = [&](auto &&at, float &mean) {   // at(i, u): the row; returns 1 / sqrt(statistic + eps)
+        mean = a.centered ? over_row(at) * inv_w : 0.f;
+        const float ss = over_row([&](int i, int u) {
+            const float d = at(i, u) - mean;
+            return d * d;
+        });
+        return 1.0f / sqrtf(ss * inv_w + a.eps);
+    };
+    if constexpr (HELD > 0) {
+#pragma unroll
+        for (int u = 0; u < PT; u++) {
+            const int i = threadIdx.x + 256 * u;
+            held[u] = i < W ? y_at(i) : 0.f;
+        }
+    }
+    float mean;
+    float inv = norm_of([&](int i, int u) { return HELD ? held[u] : y_at(i); }, mean);
+    auto update = [&](int i, float y) {
+        const float v = (a.accumulate ? x[i] : 0.f) + (y - mean) * inv * vmx_bf16_to_f32(a.w_post[i]);
+        x[i] = v;
+        return v;
+    };
+    if constexpr (HELD > 0) {
+#pragma unroll
+        for (int u = 0; u < PT; u++) {
+            const int i = threadIdx.x + 256 * u;
+            if (i < W) held[u] = update(i, held[u]);
+        }
+    } else {
+        for (int i = threadIdx.x; i < W; i += 256) update(i, y_at(i));
+    }
+    if (!a.w_next) return;
+    inv = norm_of([&](int i, int u) { return HELD ? held[u] : x[i]; }, mean);
+    auto store = [&](int i, float v) {
+        v = (v - mean) * inv * vmx_bf16_to_f32(a.w_next[i]);
+        if (a.h_f32) ((float *)a.h)[(int64_t)t * W + i] = v;
+        else ((uint16_t *)a.h)[(int64_t)t * W + i] = vmx_f32_to_bf16(v);
+    };
+    if constexpr (HELD > 0) {
+#pragma unroll
+        for (int u = 0; u < PT; u++) {
+            const int i = threadIdx.x + 256 * u;
+            if (i < W) store(i, held[u]);
+        }
+    } else {
+        for (int i = threadIdx.x; i < W; i += 256) store(i, x[i]);
     }
 }
 
@@ -205,14 +310,15 @@ __global__ __launch_bounds__(256) void embed_scaled_f32_kernel(float *__restrict
     for (int i = threadIdx.x; i < width; i += 256) x[(int64_t)t * width + i] = vmx_bf16_to_f32(embed[(int64_t)id * width + i]) * scale;
 }
 
-// act[r, j] = silu(gu[r, j]) * gu[r, ff + j]: the gated activation between the two products of a feed-forward whose gate and up
-// projections were computed as one product
-__global__ __launch_bounds__(256) void glu_silu_kernel(void *__restrict__ act, int act_f32, const float *__restrict__ gu, int ff) {
+// act[r, j] = f(gu[r, j]) * gu[r, ff + j]: the gated activation between the two products of a feed-forward whose gate and up
+// projections were computed as one product; f = silu or (GELU) the tanh form of gelu
+template <bool GELU> __global__ __launch_bounds__(256) void glu_kernel(void *__restrict__ act, int act_f32, const float *__restrict__ gu, int ff) {
     const int64_t r = blockIdx.x;             // rows on x: a prompt's (token, expert) pairs can pass the 65535 of the other axes
     const int j = blockIdx.y * 256 + threadIdx.x;
     if (j >= ff) return;
     const float g = gu[r * 2 * ff + j], u = gu[r * 2 * ff + ff + j];
-    const float v = g / (1.0f + expf(-g)) * u;
+    const float f = GELU ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) : g / (1.0f + expf(-g));
+    const float v = f * u;
     if (act_f32) ((float *)act)[r * ff + j] = v;
     else ((uint16_t *)act)[r * ff + j] = vmx_f32_to_bf16(v);
 }
@@ -238,6 +344,31 @@ __global__ __launch_bounds__(256) void scale_softcap_kernel(float *__restrict__ 
 
 }  // namespace
 
+extern "C" int vmx_rotation_steps(const vmx_rotation *rot, float *steps, float *mul) {
+    VMX_REQUIRE(rot && steps && mul, "rotation_steps: null pointer");
+    const vmx_rotation &r = *rot;
+    VMX_REQUIRE(r.dims >= 2 && r.dims % 2 == 0 && r.base > 1.0, "rotation_steps: %d rotated coordinates, base %g", r.dims, r.base);
+    const int half = r.dims / 2;
+    *mul = 1.f;
+    double lo = 0, hi = 0;
+    if (r.factor > 0.0) {
+        VMX_REQUIRE(r.original > 0.0 && r.fast > 0.0 && r.slow > 0.0, "rotation_steps: bad stretch constants");
+        auto idx = [&](double turns) { return r.dims * log(r.original / (2.0 * M_PI * turns)) / (2.0 * log(r.base)); };
+        lo = std::max(floor(idx(r.fast)), 0.0);
+        hi = std::min(ceil(idx(r.slow)), (double)(r.dims - 1));
+        *mul = (float)(0.1 * log(r.factor) + 1.0);
+    }
+    for (int i = 0; i < half; i++) {
+        double f = pow(r.base, -2.0 * i / r.dims);
+        if (r.factor > 0.0) {
+            const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            f = f / r.factor * ramp + f * (1.0 - ramp);
+        }
+        steps[i] = (float)f;
+    }
+    return VMX_OK;
+}
+
 int vmx_embed_scaled_f32(float *x, const uint16_t *embed, const int32_t *tokens, int T, int width, int vocab, float scale, hipStream_t st) {
     hipLaunchKernelGGL(embed_scaled_f32_kernel, dim3(T), dim3(256), 0, st, x, embed, tokens, width, vocab, scale);
     VMX_CHECK_LAUNCH("embed");
@@ -246,16 +377,44 @@ int vmx_embed_scaled_f32(float *x, const uint16_t *embed, const int32_t *tokens,
 
 int vmx_glu_silu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st) {
     if (rows <= 0) return VMX_OK;
-    hipLaunchKernelGGL(glu_silu_kernel, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff);
+    hipLaunchKernelGGL(glu_kernel<false>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff);
     VMX_CHECK_LAUNCH("glu silu");
+    return VMX_OK;
+}
+
+int vmx_glu_gelu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st) {
+    if (rows <= 0) return VMX_OK;
+    hipLaunchKernelGGL(glu_kernel<true>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff);
+    VMX_CHECK_LAUNCH("glu gelu");
     return VMX_OK;
 }
 
 int vmx_rms_norm_f32in(void *out, int out_f32, const float *x, const int32_t *rows, const uint16_t *w, int w_scalar, int width, float eps,
                        int n, hipStream_t st) {
     if (n <= 0) return VMX_OK;
-    hipLaunchKernelGGL(rms_norm_f32in_kernel, dim3(n), dim3(256), 0, st, out, out_f32, x, rows, w, w_scalar, width, eps);
+    hipLaunchKernelGGL(row_norm_f32in_kernel<false>, dim3(n), dim3(256), 0, st, out, out_f32, x, rows, w, w_scalar, width, eps);
     VMX_CHECK_LAUNCH("rms norm");
+    return VMX_OK;
+}
+
+int vmx_layer_norm_f32in(void *out, int out_f32, const float *x, const int32_t *rows, const uint16_t *w, int width, float eps, int n, hipStream_t st) {
+    if (n <= 0) return VMX_OK;
+    hipLaunchKernelGGL(row_norm_f32in_kernel<true>, dim3(n), dim3(256), 0, st, out, out_f32, x, rows, w, 0, width, eps);
+    VMX_CHECK_LAUNCH("layer norm");
+    return VMX_OK;
+}
+
+int vmx_sandwich_norm(const VmxSandwich &a, int n, hipStream_t st) {
+    VMX_REQUIRE(a.x && a.w_post && a.width >= 1 && (a.embed ? a.tokens && a.vocab >= 1 : a.y != nullptr), "sandwich norm: null pointer");
+    VMX_REQUIRE(!a.w_next || a.h, "sandwich norm: the next norm needs its output rows");
+    VMX_REQUIRE(!a.pair_rows || (a.pair_w && a.top >= 1), "sandwich norm: expert results need their weights");
+    if (n <= 0) return VMX_OK;
+    if (a.width <= 256) hipLaunchKernelGGL(sandwich_norm_kernel<1>, dim3(n), dim3(256), 0, st, a);
+    else if (a.width <= 1024) hipLaunchKernelGGL(sandwich_norm_kernel<4>, dim3(n), dim3(256), 0, st, a);
+    else if (a.width <= 2048) hipLaunchKernelGGL(sandwich_norm_kernel<8>, dim3(n), dim3(256), 0, st, a);
+    else if (a.width <= 4096) hipLaunchKernelGGL(sandwich_norm_kernel<16>, dim3(n), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL(sandwich_norm_kernel<0>, dim3(n), dim3(256), 0, st, a);
+    VMX_CHECK_LAUNCH("sandwich norm");
     return VMX_OK;
 }
 

@@ -204,6 +204,9 @@ struct VmxLinear {
 };
 int vmx_linear_launch(const VmxLinear &p, hipStream_t st);
 
+// latent_attn.hip: out[h][r][d] = in[h][d][r], the key up-projection turned for q_abs = U_h^T q_h
+int vmx_latent_transpose_heads(uint16_t *out, const uint16_t *in, int heads, int dim, int kv_rank, hipStream_t st);
+
 // packed_ops.hip: what the packed-step executors share
 // A device allocation owned by an executor (host-side handle).
 struct VmxBuf {
@@ -231,6 +234,30 @@ constexpr int VMX_MOE_FEW_PAIRS = 16;      // most (token, slot) pairs of a step
 // out[r] = x[rows ? rows[r] : r] / sqrt(mean(x^2) + eps) * w (w_scalar: w[0] for every column); out f32 or bf16 [n, width]
 int vmx_rms_norm_f32in(void *out, int out_f32, const float *x, const int32_t *rows, const uint16_t *w, int w_scalar, int width, float eps,
                        int n, hipStream_t st);
+// the same with the row's mean taken off first (layer norm, a gain per column)
+int vmx_layer_norm_f32in(void *out, int out_f32, const float *x, const int32_t *rows, const uint16_t *w, int width, float eps, int n, hipStream_t st);
+// Both norms around a residual sum in one pass: x[t] <- (accumulate ? x[t] : 0) + N(y[t]) * w_post, h[t] = N(x[t]) * w_next; N a layer
+// norm (centered) or an RMS norm over `width` columns.  y[t] is, in this order: row tokens[t] of the bf16 table `embed`; the sum
+// over s < top of pair_w[t top + s] * (row pair_rows[t top + s] of y) + sigmoid(shared_gate[t ld]) * shared[t] (shared, its gate:
+// optional); row t of y.
+struct VmxSandwich {
+    float *x = nullptr;
+    const float *y = nullptr;
+    const uint16_t *embed = nullptr;
+    const int32_t *tokens = nullptr;
+    int vocab = 0;
+    const int32_t *pair_rows = nullptr;
+    const float *pair_w = nullptr;
+    int top = 0;
+    const float *shared = nullptr, *shared_gate = nullptr;
+    int64_t ld_shared_gate = 0;
+    int accumulate = 1, centered = 1;
+    const uint16_t *w_post = nullptr, *w_next = nullptr;   // w_next NULL: only the sum
+    void *h = nullptr;
+    int h_f32 = 0, width = 0;
+    float eps = 0.f;
+};
+int vmx_sandwich_norm(const VmxSandwich &a, int n, hipStream_t st);
 int vmx_zero_f32(float *p, int64_t n, hipStream_t st);
 // Norm after the sum over `groups` equal consecutive parts of the row: v = acc[t], each part divided by its own sqrt(mean^2 + eps),
 // times w (w NULL: v = acc[t] as it is); x[t] = v, h[t] = v (f32 or bf16), acc[t] = alpha * v
@@ -252,6 +279,8 @@ int vmx_argmax_f32_rows(int32_t *out, unsigned long long *keys, const float *log
 int vmx_embed_scaled_f32(float *x, const uint16_t *embed, const int32_t *tokens, int T, int width, int vocab, float scale, hipStream_t st);
 // act[r, j] = silu(gu[r, j]) * gu[r, ff + j], gu f32 [rows, 2 ff], act f32 or bf16 [rows, ff]
 int vmx_glu_silu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st);
+// act[r, j] = gelu(gu[r, j]) * gu[r, ff + j], the tanh form of gelu
+int vmx_glu_gelu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st);
 // out[t] = [a[t] | b[t]]: two f32 rows of `width` numbers side by side, stored in f32 or bf16
 int vmx_concat2_rows(void *out, int out_f32, const float *a, const float *b, int T, int width, hipStream_t st);
 // x <- cap * tanh(x * scale / cap) over n numbers (cap 0: x * scale)
