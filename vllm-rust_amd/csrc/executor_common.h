@@ -38,6 +38,8 @@ inline int vmx_upload_rotation(const vmx_rotation &r, VmxBuf &steps, float &mul)
     return VMX_OK;
 }
 
+inline void vmx_erase_name(std::vector<std::string> &v, const std::string &name) { v.erase(std::remove(v.begin(), v.end(), name), v.end()); }
+
 // Checkpoint name -> destination (rows of a fused projection, or a buffer of its own), and which names are still to come.
 struct VmxTensorTable {
     struct Seg {
@@ -55,9 +57,7 @@ struct VmxTensorTable {
             if (t.first == name) return &t.second;
         return nullptr;
     }
-    void loaded(const std::string &name) {
-        missing.erase(std::remove(missing.begin(), missing.end(), name), missing.end());
-    }
+    void loaded(const std::string &name) { vmx_erase_name(missing, name); }
 };
 
 // Routing results of a step and the blocks its experts run as.  Up to VMX_MOE_FEW_PAIRS pairs: every pair is its own 16-row block

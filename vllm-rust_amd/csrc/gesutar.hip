@@ -12,11 +12,9 @@
 // router, rotations, scores and softmax are f32 in both modes; in VMX_BF16 mode the linears take bf16 operands (f32
 // accumulation) and the cache holds bf16, in VMX_F32 mode every product is a true f32 product and the cache holds f32.
 // Like the other executors the forward call allocates nothing, reads nothing back and is graph-capturable.
-#include "vmx_kernels.h"
+#include "executor_common.h"
 #include <float.h>
 #include <math.h>
-#include <string>
-#include <vector>
 
 namespace {
 
@@ -37,8 +35,8 @@ struct vmx_gesutar {
     Buf embed, bigram, final_norm, head;
     std::vector<std::string> missing;
     // step workspaces, sized for max_tokens
-    Buf x, h, fused, qabs, qrot, olat, attn, attn_ws, argmax_keys, few_pairs, rlogits, topw, topi, sorted, blk_expert, total, inv, act, ydown, sact, sout, hsel;
-    int sorted_cap = 0;
+    VmxExpertBlocks blocks;
+    Buf x, h, fused, qabs, qrot, olat, attn, attn_ws, argmax_keys, rlogits, act, ydown, sact, sout, hsel;
     bool f32() const { return cfg.dtype == VMX_F32; }
     size_t esz() const { return f32() ? 4 : 2; }
 };
@@ -63,20 +61,6 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(float *__restrict__ x
     }
 }
 
-int upload(Buf &b, size_t offset, const void *data, size_t bytes, hipStream_t st) {
-    VMX_CHECK_HIP(hipMemcpyAsync((char *)b.p + offset, data, bytes, hipMemcpyDefault, st));
-    VMX_CHECK_HIP(hipStreamSynchronize(st));
-    return VMX_OK;
-}
-
-void erase_name(std::vector<std::string> &v, const std::string &n) {
-    for (size_t i = 0; i < v.size(); i++)
-        if (v[i] == n) {
-            v.erase(v.begin() + i);
-            return;
-        }
-}
-
 }  // namespace
 
 extern "C" int vmx_gesutar_create(const vmx_gesutar_config *cfg, const vmx_gesutar_layer_config *layer_cfgs, vmx_gesutar **out) {
@@ -91,7 +75,7 @@ extern "C" int vmx_gesutar_create(const vmx_gesutar_config *cfg, const vmx_gesut
     m->cfg = c;
     m->layers.resize(c.num_layers);
     const size_t T = c.max_tokens, W = c.width;
-    size_t maxr = 0, nf = 0, hr = 0, hrd = 0, hv = 0, ne = 1, pairs = 0, eff = 0, sff = 0, cap = 0;
+    size_t maxr = 0, nf = 0, hr = 0, hrd = 0, hv = 0, ne = 1, eff = 0, sff = 0;
     int rc = VMX_OK;
 #define GA(buf, n)                       \
     do {                                 \
@@ -161,8 +145,7 @@ extern "C" int vmx_gesutar_create(const vmx_gesutar_config *cfg, const vmx_gesut
                 L.missing.push_back(pre + "mlp.shared.down");
             }
             ne = std::max(ne, (size_t)lc.experts);
-            pairs = std::max(pairs, T * lc.top);
-            cap = std::max(cap, std::max(T * lc.top + (size_t)lc.experts * 63, (size_t)VMX_MOE_FEW_PAIRS * 16));
+            m->blocks.reserve(T, lc.experts, lc.top);
             eff = std::max(eff, (size_t)lc.expert_ff);
             sff = std::max(sff, (size_t)lc.shared_ff);
         } else if (lc.mlp != VMX_MLP_NONE) {
@@ -176,6 +159,7 @@ extern "C" int vmx_gesutar_create(const vmx_gesutar_config *cfg, const vmx_gesut
         hrd = std::max(hrd, (size_t)lc.heads * lc.rot_dim);
         hv = std::max(hv, ng);
     }
+    const size_t cap = m->blocks.rows;
     GA(m->embed, (size_t)c.vocab * W * 2);
     GA(m->bigram, (size_t)(c.bigram_buckets + 1) * W * 2);
     GA(m->final_norm, W * 2);
@@ -192,34 +176,13 @@ extern "C" int vmx_gesutar_create(const vmx_gesutar_config *cfg, const vmx_gesut
     GA(m->attn_ws, (size_t)24576 * (maxr + 2) * 4);   // key partitions of launches with few rows: tokens x heads x partitions < 24576
     GA(m->attn, T * hv * m->esz());
     GA(m->argmax_keys, T * ((size_t)c.vocab / VMX_ARGMAX_CHUNK + 1) * 8);
-    GA(m->few_pairs, (size_t)(2 * VMX_MOE_FEW_PAIRS * 16 + VMX_MOE_FEW_PAIRS + 1) * 4);
     GA(m->rlogits, T * ne * 4);
-    GA(m->topw, (pairs + 1) * 4);
-    GA(m->topi, (pairs + 1) * 4);
-    GA(m->sorted, (cap + 1) * 4);
-    GA(m->blk_expert, (cap / 16 + 2) * 4);
-    GA(m->total, 16);
-    GA(m->inv, (pairs + 1) * 4);
     GA(m->act, (cap + 1) * eff * m->esz());
     GA(m->ydown, (cap + 1) * W * 4);
     GA(m->sact, T * (sff + 1) * m->esz());
     GA(m->sout, T * W * 4);
 #undef GA
-    if (!rc) {
-        // decode steps with a handful of (token, slot) pairs skip the sort: pair p is its own 16-row block (row 16 p)
-        std::vector<int32_t> fp(2 * VMX_MOE_FEW_PAIRS * 16 + VMX_MOE_FEW_PAIRS + 1);
-        for (int i = 0; i < VMX_MOE_FEW_PAIRS * 16; i++) {
-            fp[i] = i % 16 == 0 ? i / 16 : 0x7fffffff;                        // gathered rows of the up product: pair index or padding
-            fp[VMX_MOE_FEW_PAIRS * 16 + i] = i % 16 == 0 ? i : 0x7fffffff;            // rows of the down product: themselves or padding
-        }
-        for (int p = 0; p < VMX_MOE_FEW_PAIRS; p++) fp[2 * VMX_MOE_FEW_PAIRS * 16 + p] = 16 * p;   // where pair p's result lies
-        fp[2 * VMX_MOE_FEW_PAIRS * 16 + VMX_MOE_FEW_PAIRS] = 0x7fffffff;                       // "total rows": never cuts
-        if (hipMemcpy(m->few_pairs.p, fp.data(), fp.size() * 4, hipMemcpyHostToDevice) != hipSuccess) {
-            vmx_set_error("gesutar_create: upload failed");
-            rc = VMX_ELAUNCH;
-        }
-    }
-    m->sorted_cap = (int)cap;
+    if (!rc) rc = m->blocks.alloc();
     if (rc) {
         vmx_gesutar_destroy(m);
         return rc;
@@ -234,9 +197,10 @@ extern "C" void vmx_gesutar_destroy(vmx_gesutar *m) {
         for (Buf *b : {&L.norm1, &L.norm2, &L.wfused, &L.dkv_norm, &L.uk, &L.uk_t, &L.uv, &L.sink, &L.wo, &L.router, &L.eup, &L.edown, &L.sup, &L.sdown,
                        &L.inv_freq, &L.cache})
             b->release();
-    for (Buf *b : {&m->embed, &m->bigram, &m->final_norm, &m->head, &m->x, &m->h, &m->fused, &m->qabs, &m->qrot, &m->olat, &m->attn, &m->attn_ws, &m->argmax_keys, &m->few_pairs, &m->rlogits,
-                   &m->topw, &m->topi, &m->sorted, &m->blk_expert, &m->total, &m->inv, &m->act, &m->ydown, &m->sact, &m->sout, &m->hsel})
+    for (Buf *b : {&m->embed, &m->bigram, &m->final_norm, &m->head, &m->x, &m->h, &m->fused, &m->qabs, &m->qrot, &m->olat, &m->attn, &m->attn_ws, &m->argmax_keys, &m->rlogits,
+                   &m->act, &m->ydown, &m->sact, &m->sout, &m->hsel})
         b->release();
+    m->blocks.release();
     delete m;
 }
 
@@ -293,14 +257,14 @@ extern "C" int vmx_gesutar_load_tensor(vmx_gesutar *m, const char *name, const v
     VMX_REQUIRE(dst, "gesutar_load_tensor: unknown tensor `%s`", name);
     VMX_REQUIRE(bytes == need, "gesutar_load_tensor: `%s`: expected %zu bytes of bf16, got %zu", name, need, bytes);
     if (bytes > 0) {
-        if (int rc = upload(*dst, off, data, bytes, st)) return rc;
+        if (int rc = vmx_upload(*dst, off, data, bytes, st)) return rc;
         if (n.size() > 7 && n.compare(n.size() - 7, 7, ".mix.uk") == 0) {
             Layer &L = m->layers[atoi(n.substr(1).c_str())];
             if (int rc = vmx_latent_transpose_heads(L.uk_t.as<uint16_t>(), L.uk.as<uint16_t>(), L.c.heads, L.c.dim, L.c.kv_rank, st)) return rc;
             VMX_CHECK_HIP(hipStreamSynchronize(st));
         }
     }
-    erase_name(*missing, n);
+    vmx_erase_name(*missing, n);
     return VMX_OK;
 }
 
@@ -386,6 +350,7 @@ extern "C" int vmx_gesutar_forward(vmx_gesutar *m, const int32_t *tokens, const 
         // ---- feed-forward: mixture of experts
         if (lc.mlp == VMX_MLP_MOE) {
             const int E = lc.experts, k = lc.top, ff = lc.expert_ff, pairs = T * k;
+            VmxExpertBlocks &b = m->blocks;
             if (int rc = vmx_rms_norm_f32in(m->h.p, f32, x, nullptr, L.norm2.as<uint16_t>(), 0, W, c.norm_eps, T, st)) return rc;
             VmxLinear r;   // router logits: always a true f32 product
             r.A = m->h.p, r.a_f32 = f32, r.lda = W;
@@ -395,38 +360,23 @@ extern "C" int vmx_gesutar_forward(vmx_gesutar *m, const int32_t *tokens, const 
             if (int rc = vmx_linear_launch(r, st)) return rc;
             // logits and routing stay two launches: one workgroup per token doing both walks K once per 16 experts in sequence
             // (21.5 us at one row of 2048 against 10.3 + 5.7 us for the pair)
-            if (int rc = vmx_grouped_topk_router(m->rlogits.as<float>(), m->topw.as<float>(), m->topi.as<int32_t>(), T, E, k, lc.groups,
+            if (int rc = vmx_grouped_topk_router(m->rlogits.as<float>(), b.topw.as<float>(), b.topi.as<int32_t>(), T, E, k, lc.groups,
                                                  lc.keep_groups, lc.router_scale, st))
                 return rc;
-            const bool few = pairs <= VMX_MOE_FEW_PAIRS;   // every pair its own block: no sort, an expert's weights are read once per pair
-            const int br = few ? 16 : (pairs >= 32 * E ? 64 : 16);
-            const int cap = few ? pairs * 16 : pairs + E * (br - 1);
-            const int32_t *fp = m->few_pairs.as<int32_t>();
-            const int32_t *up_rows = few ? fp : m->sorted.as<int32_t>(), *down_rows = few ? fp + VMX_MOE_FEW_PAIRS * 16 : nullptr;
-            const int32_t *blk = few ? m->topi.as<int32_t>() : m->blk_expert.as<int32_t>();
-            const int32_t *total = few ? fp + 2 * VMX_MOE_FEW_PAIRS * 16 + VMX_MOE_FEW_PAIRS : m->total.as<int32_t>();
-            const int32_t *inv = few ? fp + 2 * VMX_MOE_FEW_PAIRS * 16 : m->inv.as<int32_t>();
-            if (!few) {
-                if (int rc = vmx_moe_align_block_size(m->topi.as<int32_t>(), m->sorted.as<int32_t>(), m->blk_expert.as<int32_t>(),
-                                                      m->total.as<int32_t>(), pairs, E, br, cap, st))
-                    return rc;
-                if (int rc = vmx_moe_inverse(m->inv.as<int32_t>(), m->sorted.as<int32_t>(), m->total.as<int32_t>(), pairs, cap, st)) return rc;
-            }
+            if (int rc = b.plan(pairs, E, st)) return rc;
             VmxLinear u;   // act = relu(W_up[e] h)^2 over the pairs' rows
             u.A = m->h.p, u.a_f32 = f32, u.lda = W;
             u.W = L.eup.as<uint16_t>(), u.w_sn = W, u.w_sk = 1;
             u.C = m->act.p, u.c_f32 = f32, u.ldc = ff;
-            u.M = cap, u.N = ff, u.K = W, u.exact = f32, u.epilogue = VMX_EP_RELU2;
-            u.row_ids = up_rows, u.row_div = k, u.row_limit = pairs;
-            u.block_expert = blk, u.expert_stride = (int64_t)ff * W, u.block_rows = br, u.total_rows = total;
+            u.N = ff, u.K = W, u.exact = f32, u.epilogue = VMX_EP_RELU2;
+            b.first(u, pairs, k, (int64_t)ff * W);
             if (int rc = vmx_linear_launch(u, st)) return rc;
             VmxLinear d;   // y = W_down[e] act
             d.A = m->act.p, d.a_f32 = f32, d.lda = ff;
             d.W = L.edown.as<uint16_t>(), d.w_sn = ff, d.w_sk = 1;
             d.C = m->ydown.p, d.c_f32 = 1, d.ldc = W;
-            d.M = cap, d.N = W, d.K = ff, d.exact = f32;
-            d.row_ids = down_rows, d.row_div = 1, d.row_limit = cap;
-            d.block_expert = blk, d.expert_stride = (int64_t)ff * W, d.block_rows = br, d.total_rows = total;
+            d.N = W, d.K = ff, d.exact = f32;
+            b.second(d, (int64_t)ff * W);
             if (int rc = vmx_linear_launch(d, st)) return rc;
             const float *shared = nullptr;
             if (lc.shared_ff > 0) {
@@ -444,7 +394,7 @@ extern "C" int vmx_gesutar_forward(vmx_gesutar *m, const int32_t *tokens, const 
                 if (int rc = vmx_linear_launch(sd, st)) return rc;
                 shared = m->sout.as<float>();
             }
-            if (int rc = vmx_moe_combine_f32(x, m->ydown.as<float>(), inv, m->topw.as<float>(), k, shared, nullptr, 0, T, W, st)) return rc;
+            if (int rc = vmx_moe_combine_f32(x, m->ydown.as<float>(), b.pair_rows, b.topw.as<float>(), k, shared, nullptr, 0, T, W, st)) return rc;
         }
         if (layer_trace)
             VMX_CHECK_HIP(hipMemcpyAsync(layer_trace + (size_t)li * T * W, x, (size_t)T * W * 4, hipMemcpyDeviceToDevice, st));

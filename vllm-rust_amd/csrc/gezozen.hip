@@ -24,24 +24,15 @@
 // VMX_BF16 mode) and the next alpha * x.  The stream, norms, router, positions and angles, scores, softmax, decays, gates of the
 // recurrences and their state are f32 in both modes; VMX_BF16 rounds the operands of the linears and the cache rows to bf16,
 // VMX_F32 multiplies in true f32 everywhere.  The forward call allocates nothing, reads nothing back and is graph-capturable.
-#include "vmx_kernels.h"
+#include "executor_common.h"
 #include <math.h>
-#include <algorithm>
-#include <string>
-#include <vector>
 
 namespace {
 
 using Buf = VmxBuf;
+using Seg = VmxTensorTable::Seg;
 
-int pad8(int n) { return (n + 7) & ~7; }
-
-struct Seg {       // where a checkpoint tensor lands: rows of a fused projection, or a buffer of its own
-    Buf *buf = nullptr;
-    size_t offset = 0, bytes = 0;
-};
-
-struct Layer {
+struct Layer : VmxTensorTable {
     vmx_gezozen_layer_config c;
     Buf norm1, norm2, wfused, bias, wfused2, bias2;
     Buf qnorm, knorm, wo, rot_steps, kcache, vcache;                                // attention
@@ -52,12 +43,6 @@ struct Layer {
     int nf = 0, q_off = 0, k_off = 0, v_off = 0, rq_off = 0, rk_off = 0, rv_off = 0, g_off = 0, a1_off = 0, b_off = 0, a_off = 0, rg1_off = 0;
     int nf2 = 0, sgu_off = 0, sg_off = 0, rg2_off = 0;
     int rh = 0, rqk = 0, rd = 0, rv = 0;   // the recurrence as it runs: value heads, query/key heads, key size, value size
-    std::vector<std::pair<std::string, Seg>> tensors;   // checkpoint name (without the layer prefix) -> destination
-    std::vector<std::string> missing;
-    void want(const std::string &name, Buf *b, size_t off, size_t bytes) {
-        tensors.push_back({name, Seg{b, off, bytes}});
-        missing.push_back(name);
-    }
 };
 
 }  // namespace
@@ -68,50 +53,11 @@ struct vmx_gezozen {
     Buf embed, final_norm, head;
     std::vector<std::string> missing;
     Buf x, acc, h, hsel, fused, qbuf, attn, attn_ws, conv, dec, dro, rec, argmax_keys;
-    Buf few_pairs, rlogits, topw, topi, sorted, blk_expert, total, inv, gu, act, ydown, sact, sout;
+    VmxExpertBlocks blocks;
+    Buf rlogits, gu, act, ydown, sact, sout;
     bool f32() const { return cfg.dtype == VMX_F32; }
     size_t esz() const { return f32() ? 4 : 2; }
 };
-
-namespace {
-
-int upload(Buf &b, size_t offset, const void *data, size_t bytes, hipStream_t st) {
-    VMX_CHECK_HIP(hipMemcpyAsync((char *)b.p + offset, data, bytes, hipMemcpyDefault, st));
-    VMX_CHECK_HIP(hipStreamSynchronize(st));
-    return VMX_OK;
-}
-
-void erase_name(std::vector<std::string> &v, const std::string &n) {
-    for (size_t i = 0; i < v.size(); i++)
-        if (v[i] == n) {
-            v.erase(v.begin() + i);
-            return;
-        }
-}
-
-int alloc_zero(Buf &b, size_t n) {
-    if (int rc = b.alloc(n)) return rc;
-    VMX_CHECK_HIP(hipMemset(b.p, 0, n ? n : 16));
-    return VMX_OK;
-}
-
-bool rotation_ok(const vmx_rotation &r, int head_dim) {
-    if (r.dims == 0) return true;
-    if (r.dims < 0 || r.dims % 2 || r.dims > head_dim || !(r.base > 1.0)) return false;
-    return r.factor == 0.0 || (r.factor > 0.0 && r.original > 0.0 && r.fast > 0.0 && r.slow > 0.0);
-}
-
-int upload_rotation(const vmx_rotation &r, Buf &steps, float &mul) {
-    mul = 1.f;
-    if (r.dims <= 0) return VMX_OK;
-    std::vector<float> f(r.dims / 2);
-    if (int rc = vmx_rotation_steps(&r, f.data(), &mul)) return rc;
-    if (int rc = steps.alloc(f.size() * 4)) return rc;
-    VMX_CHECK_HIP(hipMemcpy(steps.p, f.data(), f.size() * 4, hipMemcpyHostToDevice));
-    return VMX_OK;
-}
-
-}  // namespace
 
 extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezozen_layer_config *layer_cfgs, vmx_gezozen **out) {
     VMX_REQUIRE(cfg && layer_cfgs && out, "gezozen_create: null pointer");
@@ -127,11 +73,11 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
     m->cfg = c;
     m->layers.resize(c.num_layers);
     const size_t T = c.max_tokens, W = c.width, rows = (size_t)c.num_blocks * c.block_size;
-    size_t attn_ws = 16, nf = 8, hd = 1, hv = 1, convc = 1, rhd = 1, rhv = 1, ne = 1, pairs = 0, cap = (size_t)VMX_MOE_FEW_PAIRS * 16, eff = 1, sff = 1;
+    size_t attn_ws = 16, nf = 8, hd = 1, hv = 1, convc = 1, rhd = 1, rhv = 1, ne = 1, eff = 1, sff = 1;
     int rc = VMX_OK;
-#define GA(buf, n)                        \
-    do {                                  \
-        if (!rc) rc = alloc_zero(buf, n); \
+#define GA(buf, n)                            \
+    do {                                      \
+        if (!rc) rc = vmx_alloc_zero(buf, n); \
     } while (0)
 #define BAD(...)                    \
     {                               \
@@ -152,7 +98,7 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
         int at = 0;
         auto seg = [&](int n) {
             const int o = at;
-            at = pad8(at + n);
+            at = vmx_pad8(at + n);
             return o;
         };
         L.want("norm1", &L.norm1, 0, W * 2);
@@ -161,11 +107,11 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
         if (two_sided) {
             const bool gla = lc.mixer == VMX_MIXER_ATTENTION_GLA;
             if (lc.window < 0 || lc.softcap < 0.f) BAD("gezozen_create: layer %d: bad attention mask or soft cap", li);
-            if (!rotation_ok(lc.rot, lc.dim)) BAD("gezozen_create: layer %d: bad rotation of the attention (%d coordinates in heads of %d)", li, lc.rot.dims, lc.dim);
+            if (!vmx_rotation_ok(lc.rot, lc.dim)) BAD("gezozen_create: layer %d: bad rotation of the attention (%d coordinates in heads of %d)", li, lc.rot.dims, lc.dim);
             if (lc.r_heads < 1 || lc.r_dim < 1 || lc.r_dim > 256 || lc.r_vdim < 1)
                 BAD("gezozen_create: layer %d: bad sizes of the recurrent side (heads %d, dim %d, vdim %d)", li, lc.r_heads, lc.r_dim, lc.r_vdim);
             if (gla && (!(lc.tau > 0.f) || lc.decay_rank < 1)) BAD("gezozen_create: layer %d: bad decay constants (tau %g, rank %d)", li, lc.tau, lc.decay_rank);
-            if (!gla && (!lc.decay || !rotation_ok(lc.r_rot, lc.r_dim))) BAD("gezozen_create: layer %d: retention needs its decays and a valid rotation", li);
+            if (!gla && (!lc.decay || !vmx_rotation_ok(lc.r_rot, lc.r_dim))) BAD("gezozen_create: layer %d: retention needs its decays and a valid rotation", li);
             const size_t RH = lc.r_heads, RD = lc.r_dim, RV = lc.r_vdim;
             L.rh = L.rqk = lc.r_heads, L.rd = lc.r_dim, L.rv = lc.r_vdim;
             L.q_off = seg(H * D);
@@ -214,9 +160,9 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
             } else {
                 GA(L.decay, RH * 4);
                 if (!rc && hipMemcpy(L.decay.p, lc.decay, RH * 4, hipMemcpyHostToDevice) != hipSuccess) BAD("gezozen_create: upload failed");
-                if (!rc) rc = upload_rotation(lc.r_rot, L.r_rot_steps, L.r_rot_mul);
+                if (!rc) rc = vmx_upload_rotation(lc.r_rot, L.r_rot_steps, L.r_rot_mul);
             }
-            if (!rc) rc = upload_rotation(lc.rot, L.rot_steps, L.rot_mul);
+            if (!rc) rc = vmx_upload_rotation(lc.rot, L.rot_steps, L.rot_mul);
             attn_ws = std::max(attn_ws, vmx_window_attention_workspace_bytes((int)T, lc.heads, lc.vdim));
             hd = std::max(hd, H * D);
             hv = std::max(hv, H * V);
@@ -300,8 +246,7 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
                 L.want("mlp.shared.down", &L.sdown, 0, W * S * 2);
             }
             ne = std::max(ne, (size_t)lc.experts);
-            pairs = std::max(pairs, T * lc.top);
-            cap = std::max(cap, T * lc.top + (size_t)lc.experts * 63);
+            m->blocks.reserve(T, lc.experts, lc.top);
             eff = std::max(eff, (size_t)lc.expert_ff);
             sff = std::max(sff, S);
             nf = std::max(nf, (size_t)L.nf2);
@@ -313,6 +258,7 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
         nf = std::max(nf, (size_t)L.nf);
     }
 #undef BAD
+    const size_t cap = m->blocks.rows;
     GA(m->embed, (size_t)c.vocab * W * 2);
     GA(m->final_norm, W * 2);
     GA(m->head, (size_t)c.vocab * W * 2);
@@ -330,35 +276,14 @@ extern "C" int vmx_gezozen_create(const vmx_gezozen_config *cfg, const vmx_gezoz
     GA(m->dro, T * rhv * 4);
     GA(m->rec, T * rhv * m->esz());
     GA(m->argmax_keys, T * ((size_t)c.vocab / VMX_ARGMAX_CHUNK + 1) * 8);
-    GA(m->few_pairs, (size_t)(2 * VMX_MOE_FEW_PAIRS * 16 + VMX_MOE_FEW_PAIRS + 1) * 4);
     GA(m->rlogits, T * ne * 4);
-    GA(m->topw, (pairs + 1) * 4);
-    GA(m->topi, (pairs + 1) * 4);
-    GA(m->sorted, (cap + 1) * 4);
-    GA(m->blk_expert, (cap / 16 + 2) * 4);
-    GA(m->total, 16);
-    GA(m->inv, (pairs + 1) * 4);
     GA(m->gu, (cap + 1) * 2 * eff * 4);
     GA(m->act, (cap + 1) * eff * m->esz());
     GA(m->ydown, (cap + 1) * W * 4);
     GA(m->sact, T * sff * m->esz());
     GA(m->sout, T * W * 4);
 #undef GA
-    if (!rc) {
-        // decode steps with a handful of (token, slot) pairs skip the sort: pair p is its own 16-row block (row 16 p)
-        const int FP = VMX_MOE_FEW_PAIRS;
-        std::vector<int32_t> fp(2 * FP * 16 + FP + 1);
-        for (int i = 0; i < FP * 16; i++) {
-            fp[i] = i % 16 == 0 ? i / 16 : 0x7fffffff;              // gathered rows of the first product: pair index or padding
-            fp[FP * 16 + i] = i % 16 == 0 ? i : 0x7fffffff;          // rows of the second product: themselves or padding
-        }
-        for (int p = 0; p < FP; p++) fp[2 * FP * 16 + p] = 16 * p;   // where pair p's result lies
-        fp[2 * FP * 16 + FP] = 0x7fffffff;                           // "total rows": never cuts
-        if (hipMemcpy(m->few_pairs.p, fp.data(), fp.size() * 4, hipMemcpyHostToDevice) != hipSuccess) {
-            vmx_set_error("gezozen_create: upload failed");
-            rc = VMX_ELAUNCH;
-        }
-    }
+    if (!rc) rc = m->blocks.alloc();
     if (rc) {
         vmx_gezozen_destroy(m);
         return rc;
@@ -375,9 +300,10 @@ extern "C" void vmx_gezozen_destroy(vmx_gezozen *m) {
                        &L.router, &L.egu, &L.edown, &L.sdown})
             b->release();
     for (Buf *b : {&m->embed, &m->final_norm, &m->head, &m->x, &m->acc, &m->h, &m->hsel, &m->fused, &m->qbuf, &m->attn, &m->attn_ws, &m->conv, &m->dec,
-                   &m->dro, &m->rec, &m->argmax_keys, &m->few_pairs, &m->rlogits, &m->topw, &m->topi, &m->sorted, &m->blk_expert, &m->total, &m->inv,
+                   &m->dro, &m->rec, &m->argmax_keys, &m->rlogits,
                    &m->gu, &m->act, &m->ydown, &m->sact, &m->sout})
         b->release();
+    m->blocks.release();
     delete m;
 }
 
@@ -407,8 +333,8 @@ extern "C" int vmx_gezozen_load_tensor(vmx_gezozen *m, const char *name, const v
     VMX_REQUIRE(dst.buf, "gezozen_load_tensor: unknown tensor `%s`", name);
     VMX_REQUIRE(bytes == dst.bytes, "gezozen_load_tensor: `%s`: expected %zu bytes of bf16, got %zu", name, dst.bytes, bytes);
     if (bytes > 0)
-        if (int rc = upload(*dst.buf, dst.offset, data, bytes, st)) return rc;
-    erase_name(*missing, key);
+        if (int rc = vmx_upload(*dst.buf, dst.offset, data, bytes, st)) return rc;
+    vmx_erase_name(*missing, key);
     return VMX_OK;
 }
 
@@ -534,7 +460,8 @@ extern "C" int vmx_gezozen_forward(vmx_gezozen *m, const int32_t *tokens, const 
         }
         if (int rc = vmx_group_norm_post(acc, x, m->h.p, f32, L.norm1.as<uint16_t>(), c.norm_groups, W, c.norm_eps, c.postln_alpha, T, st)) return rc;
         if (lc.mlp == VMX_MLP_SIGMOID_MOE) {
-            const int E = lc.experts, k = lc.top, ff = lc.expert_ff, S = lc.shared_ff, nf2 = L.nf2, pairs = T * k, FP = VMX_MOE_FEW_PAIRS;
+            const int E = lc.experts, k = lc.top, ff = lc.expert_ff, S = lc.shared_ff, nf2 = L.nf2, pairs = T * k;
+            VmxExpertBlocks &b = m->blocks;
             {   // what reads the feed-forward's input besides the experts: shared gate | up, the shared expert's gate, residual gate 2
                 VmxLinear p;
                 p.A = m->h.p, p.a_f32 = f32, p.lda = W;
@@ -549,40 +476,25 @@ extern "C" int vmx_gezozen_forward(vmx_gezozen *m, const int32_t *tokens, const 
             r.C = m->rlogits.p, r.c_f32 = 1, r.ldc = E;
             r.M = T, r.N = E, r.K = W, r.exact = 1;
             if (int rc = vmx_linear_launch(r, st)) return rc;
-            if (int rc = vmx_topk_sigmoid(m->rlogits.as<float>(), m->topw.as<float>(), m->topi.as<int32_t>(), T, E, k, 0, stream)) return rc;
-            const bool few = pairs <= FP;   // every pair its own block: no sort
-            const int br = few ? 16 : (pairs >= 32 * E ? 64 : 16);
-            const int cap = few ? pairs * 16 : pairs + E * (br - 1);
-            const int32_t *fp = m->few_pairs.as<int32_t>();
-            const int32_t *up_rows = few ? fp : m->sorted.as<int32_t>(), *down_rows = few ? fp + FP * 16 : nullptr;
-            const int32_t *blk = few ? m->topi.as<int32_t>() : m->blk_expert.as<int32_t>();
-            const int32_t *total = few ? fp + 2 * FP * 16 + FP : m->total.as<int32_t>();
-            const int32_t *inv = few ? fp + 2 * FP * 16 : m->inv.as<int32_t>();
-            if (!few) {
-                if (int rc = vmx_moe_align_block_size(m->topi.as<int32_t>(), m->sorted.as<int32_t>(), m->blk_expert.as<int32_t>(),
-                                                      m->total.as<int32_t>(), pairs, E, br, cap, stream))
-                    return rc;
-                if (int rc = vmx_moe_inverse(m->inv.as<int32_t>(), m->sorted.as<int32_t>(), m->total.as<int32_t>(), pairs, cap, st)) return rc;
-            }
+            if (int rc = vmx_topk_sigmoid(m->rlogits.as<float>(), b.topw.as<float>(), b.topi.as<int32_t>(), T, E, k, 0, stream)) return rc;
+            if (int rc = b.plan(pairs, E, st)) return rc;
             VmxLinear u;   // gate | up of the pairs' rows in one product
             u.A = m->h.p, u.a_f32 = f32, u.lda = W;
             u.W = L.egu.as<uint16_t>(), u.w_sn = W, u.w_sk = 1;
             u.C = m->gu.p, u.c_f32 = 1, u.ldc = 2 * ff;
-            u.M = cap, u.N = 2 * ff, u.K = W, u.exact = f32;
-            u.row_ids = up_rows, u.row_div = k, u.row_limit = pairs;
-            u.block_expert = blk, u.expert_stride = (int64_t)2 * ff * W, u.block_rows = br, u.total_rows = total;
+            u.N = 2 * ff, u.K = W, u.exact = f32;
+            b.first(u, pairs, k, (int64_t)2 * ff * W);
             if (int rc = vmx_linear_launch(u, st)) return rc;
             // the router's score scales the expert's input: silu(s g) * (s u), s = score of the row's pair
-            if (int rc = vmx_glu_silu_rows_scaled(m->act.p, f32, m->gu.as<float>(), 2 * ff, ff, cap, ff, m->topw.as<float>(), up_rows, pairs, nullptr,
+            if (int rc = vmx_glu_silu_rows_scaled(m->act.p, f32, m->gu.as<float>(), 2 * ff, ff, b.cap, ff, b.topw.as<float>(), b.up_rows, pairs, nullptr,
                                                   0, st))
                 return rc;
             VmxLinear d;
             d.A = m->act.p, d.a_f32 = f32, d.lda = ff;
             d.W = L.edown.as<uint16_t>(), d.w_sn = ff, d.w_sk = 1;
             d.C = m->ydown.p, d.c_f32 = 1, d.ldc = W;
-            d.M = cap, d.N = W, d.K = ff, d.exact = f32;
-            d.row_ids = down_rows, d.row_div = 1, d.row_limit = cap;
-            d.block_expert = blk, d.expert_stride = (int64_t)ff * W, d.block_rows = br, d.total_rows = total;
+            d.N = W, d.K = ff, d.exact = f32;
+            b.second(d, (int64_t)ff * W);
             if (int rc = vmx_linear_launch(d, st)) return rc;
             if (S) {   // shared expert: its per-token gate goes onto the rows of the down projection
                 if (int rc = vmx_glu_silu_rows_scaled(m->sact.p, f32, fused + L.sgu_off, nf2, S, T, S, nullptr, nullptr, 0, fused + L.sg_off, nf2, st))
@@ -594,7 +506,7 @@ extern "C" int vmx_gezozen_forward(vmx_gezozen *m, const int32_t *tokens, const 
                 sd.M = T, sd.N = W, sd.K = S, sd.exact = f32;
                 if (int rc = vmx_linear_launch(sd, st)) return rc;
             }
-            if (int rc = vmx_moe_combine_f32(acc, m->ydown.as<float>(), inv, nullptr, k, S ? m->sout.as<float>() : nullptr, fused + L.rg2_off, nf2, T,
+            if (int rc = vmx_moe_combine_f32(acc, m->ydown.as<float>(), b.pair_rows, nullptr, k, S ? m->sout.as<float>() : nullptr, fused + L.rg2_off, nf2, T,
                                              W, st))
                 return rc;
             if (int rc = vmx_group_norm_post(acc, x, m->h.p, f32, L.norm2.as<uint16_t>(), c.norm_groups, W, c.norm_eps, c.postln_alpha, T, st)) return rc;

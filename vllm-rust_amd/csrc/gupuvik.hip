@@ -15,35 +15,20 @@
 // by the caller.  The residual stream, norms, router, scores, softmax, decays, gates and the recurrence are f32 in both modes;
 // VMX_BF16 rounds the operands of the linears and the cache rows to bf16, VMX_F32 multiplies in true f32 everywhere.
 // The forward call allocates nothing, reads nothing back and is graph-capturable.
-#include "vmx_kernels.h"
+#include "executor_common.h"
 #include <math.h>
-#include <algorithm>
-#include <string>
-#include <vector>
 
 namespace {
 
 using Buf = VmxBuf;
+using Seg = VmxTensorTable::Seg;
 
-int pad8(int n) { return (n + 7) & ~7; }
-
-struct Seg {       // where a checkpoint tensor lands: rows of the fused projection, or a buffer of its own
-    Buf *buf = nullptr;
-    size_t offset = 0, bytes = 0;
-};
-
-struct Layer {
+struct Layer : VmxTensorTable {
     vmx_gupuvik_layer_config c;
     Buf norm1, wfused, bias, wo, temp, kcache, vcache;                       // both mixers / attention
     Buf conv_taps, a_log, dt_bias, onorm, wa2, wg2, conv_state, s_state;     // channel delta
     Buf wup, wdown, router, egu, edown;                                      // feed-forward
     int nf = 0, q_off = 0, k_off = 0, v_off = 0, g_off = 0, b_off = 0, a1_off = 0, g1_off = 0, rg1_off = 0, rg2_off = 0;
-    std::vector<std::pair<std::string, Seg>> tensors;   // checkpoint name (without the layer prefix) -> destination
-    std::vector<std::string> missing;
-    void want(const std::string &name, Buf *b, size_t off, size_t bytes) {
-        tensors.push_back({name, Seg{b, off, bytes}});
-        missing.push_back(name);
-    }
 };
 
 }  // namespace
@@ -53,34 +38,11 @@ struct vmx_gupuvik {
     std::vector<Layer> layers;
     Buf embed, final_norm, head;
     std::vector<std::string> missing;
-    Buf x, h, hsel, fused, attn, attn_ws, conv, dec, gate2, dro, argmax_keys, few_pairs, rlogits, topw, topi, sorted, blk_expert, total, inv, gu, act, ydown;
+    VmxExpertBlocks blocks;
+    Buf x, h, hsel, fused, attn, attn_ws, conv, dec, gate2, dro, argmax_keys, rlogits, gu, act, ydown;
     bool f32() const { return cfg.dtype == VMX_F32; }
     size_t esz() const { return f32() ? 4 : 2; }
 };
-
-namespace {
-
-int upload(Buf &b, size_t offset, const void *data, size_t bytes, hipStream_t st) {
-    VMX_CHECK_HIP(hipMemcpyAsync((char *)b.p + offset, data, bytes, hipMemcpyDefault, st));
-    VMX_CHECK_HIP(hipStreamSynchronize(st));
-    return VMX_OK;
-}
-
-void erase_name(std::vector<std::string> &v, const std::string &n) {
-    for (size_t i = 0; i < v.size(); i++)
-        if (v[i] == n) {
-            v.erase(v.begin() + i);
-            return;
-        }
-}
-
-int alloc_zero(Buf &b, size_t n) {
-    if (int rc = b.alloc(n)) return rc;
-    VMX_CHECK_HIP(hipMemset(b.p, 0, n ? n : 16));
-    return VMX_OK;
-}
-
-}  // namespace
 
 extern "C" int vmx_gupuvik_create(const vmx_gupuvik_config *cfg, const vmx_gupuvik_layer_config *layer_cfgs, vmx_gupuvik **out) {
     VMX_REQUIRE(cfg && layer_cfgs && out, "gupuvik_create: null pointer");
@@ -94,11 +56,11 @@ extern "C" int vmx_gupuvik_create(const vmx_gupuvik_config *cfg, const vmx_gupuv
     m->cfg = c;
     m->layers.resize(c.num_layers);
     const size_t T = c.max_tokens, W = c.width, rows = (size_t)c.num_blocks * c.block_size;
-    size_t attn_ws = 16, nf = 8, hv = 1, convc = 1, hd = 1, ne = 1, pairs = 0, cap = (size_t)VMX_MOE_FEW_PAIRS * 16, eff = 1, actn = 1;
+    size_t attn_ws = 16, nf = 8, hv = 1, convc = 1, hd = 1, ne = 1, eff = 1, actn = 1;
     int rc = VMX_OK;
-#define GA(buf, n)                        \
-    do {                                  \
-        if (!rc) rc = alloc_zero(buf, n); \
+#define GA(buf, n)                            \
+    do {                                      \
+        if (!rc) rc = vmx_alloc_zero(buf, n); \
     } while (0)
 #define BAD(...)                    \
     {                               \
@@ -118,7 +80,7 @@ extern "C" int vmx_gupuvik_create(const vmx_gupuvik_config *cfg, const vmx_gupuv
         int at = 0;
         auto seg = [&](int n) {
             const int o = at;
-            at = pad8(at + n);
+            at = vmx_pad8(at + n);
             return o;
         };
         L.want("norm1", &L.norm1, 0, 2);
@@ -230,8 +192,7 @@ extern "C" int vmx_gupuvik_create(const vmx_gupuvik_config *cfg, const vmx_gupuv
                 L.want(p + "down", &L.edown, (size_t)e * one, one);
             }
             ne = std::max(ne, (size_t)lc.experts);
-            pairs = std::max(pairs, T * lc.top);
-            cap = std::max(cap, T * lc.top + (size_t)lc.experts * 63);
+            m->blocks.reserve(T, lc.experts, lc.top);
             eff = std::max(eff, (size_t)lc.expert_ff);
         } else if (lc.mlp != VMX_MLP_NONE) {
             vmx_set_error("gupuvik_create: layer %d: unknown feed-forward kind %d", li, lc.mlp);
@@ -242,6 +203,7 @@ extern "C" int vmx_gupuvik_create(const vmx_gupuvik_config *cfg, const vmx_gupuv
         hv = std::max(hv, H * V);
     }
 #undef BAD
+    const size_t cap = m->blocks.rows;
     GA(m->embed, (size_t)c.vocab * W * 2);
     GA(m->final_norm, 2);
     GA(m->head, (size_t)c.vocab * W * 2);
@@ -257,33 +219,12 @@ extern "C" int vmx_gupuvik_create(const vmx_gupuvik_config *cfg, const vmx_gupuv
     GA(m->gate2, T * hv * 4);
     GA(m->dro, T * hv * 4);
     GA(m->argmax_keys, T * ((size_t)c.vocab / VMX_ARGMAX_CHUNK + 1) * 8);
-    GA(m->few_pairs, (size_t)(2 * VMX_MOE_FEW_PAIRS * 16 + VMX_MOE_FEW_PAIRS + 1) * 4);
     GA(m->rlogits, T * ne * 4);
-    GA(m->topw, (pairs + 1) * 4);
-    GA(m->topi, (pairs + 1) * 4);
-    GA(m->sorted, (cap + 1) * 4);
-    GA(m->blk_expert, (cap / 16 + 2) * 4);
-    GA(m->total, 16);
-    GA(m->inv, (pairs + 1) * 4);
     GA(m->gu, (cap + 1) * 2 * eff * 4);
     GA(m->act, std::max((cap + 1) * eff, actn) * m->esz());
     GA(m->ydown, (cap + 1) * W * 4);
 #undef GA
-    if (!rc) {
-        // decode steps with a handful of (token, slot) pairs skip the sort: pair p is its own 16-row block (row 16 p)
-        const int FP = VMX_MOE_FEW_PAIRS;
-        std::vector<int32_t> fp(2 * FP * 16 + FP + 1);
-        for (int i = 0; i < FP * 16; i++) {
-            fp[i] = i % 16 == 0 ? i / 16 : 0x7fffffff;              // gathered rows of the first product: pair index or padding
-            fp[FP * 16 + i] = i % 16 == 0 ? i : 0x7fffffff;          // rows of the second product: themselves or padding
-        }
-        for (int p = 0; p < FP; p++) fp[2 * FP * 16 + p] = 16 * p;   // where pair p's result lies
-        fp[2 * FP * 16 + FP] = 0x7fffffff;                           // "total rows": never cuts
-        if (hipMemcpy(m->few_pairs.p, fp.data(), fp.size() * 4, hipMemcpyHostToDevice) != hipSuccess) {
-            vmx_set_error("gupuvik_create: upload failed");
-            rc = VMX_ELAUNCH;
-        }
-    }
+    if (!rc) rc = m->blocks.alloc();
     if (rc) {
         vmx_gupuvik_destroy(m);
         return rc;
@@ -299,9 +240,10 @@ extern "C" void vmx_gupuvik_destroy(vmx_gupuvik *m) {
                        &L.conv_state, &L.s_state, &L.wup, &L.wdown, &L.router, &L.egu, &L.edown})
             b->release();
     for (Buf *b : {&m->embed, &m->final_norm, &m->head, &m->x, &m->h, &m->hsel, &m->fused, &m->attn, &m->attn_ws, &m->conv, &m->dec, &m->gate2, &m->dro,
-                   &m->argmax_keys, &m->few_pairs, &m->rlogits, &m->topw, &m->topi, &m->sorted, &m->blk_expert, &m->total, &m->inv, &m->gu, &m->act,
+                   &m->argmax_keys, &m->rlogits, &m->gu, &m->act,
                    &m->ydown})
         b->release();
+    m->blocks.release();
     delete m;
 }
 
@@ -331,8 +273,8 @@ extern "C" int vmx_gupuvik_load_tensor(vmx_gupuvik *m, const char *name, const v
     VMX_REQUIRE(dst.buf, "gupuvik_load_tensor: unknown tensor `%s`", name);
     VMX_REQUIRE(bytes == dst.bytes, "gupuvik_load_tensor: `%s`: expected %zu bytes of bf16, got %zu", name, dst.bytes, bytes);
     if (bytes > 0)
-        if (int rc = upload(*dst.buf, dst.offset, data, bytes, st)) return rc;
-    erase_name(*missing, key);
+        if (int rc = vmx_upload(*dst.buf, dst.offset, data, bytes, st)) return rc;
+    vmx_erase_name(*missing, key);
     return VMX_OK;
 }
 
@@ -448,7 +390,8 @@ extern "C" int vmx_gupuvik_forward(vmx_gupuvik *m, const int32_t *tokens, const 
             d.epilogue = VMX_EP_ADD_MUL_SIGMOID, d.aux = fused + L.rg2_off, d.ldaux = nf;
             if (int rc = vmx_linear_launch(d, st)) return rc;
         } else if (lc.mlp == VMX_MLP_GLU_MOE) {
-            const int E = lc.experts, k = lc.top, ff = lc.expert_ff, pairs = T * k, FP = VMX_MOE_FEW_PAIRS;
+            const int E = lc.experts, k = lc.top, ff = lc.expert_ff, pairs = T * k;
+            VmxExpertBlocks &b = m->blocks;
             VmxLinear r;   // router logits: always a true f32 product
             r.A = m->h.p, r.a_f32 = f32, r.lda = W;
             r.W = L.router.as<uint16_t>(), r.w_sn = W, r.w_sk = 1;
@@ -456,39 +399,24 @@ extern "C" int vmx_gupuvik_forward(vmx_gupuvik *m, const int32_t *tokens, const 
             r.M = T, r.N = E, r.K = W, r.exact = 1;
             if (int rc = vmx_linear_launch(r, st)) return rc;
             // the largest `top` logits; softmax over all experts renormalised over the chosen = softmax over the chosen logits
-            if (int rc = vmx_topk_softmax(m->rlogits.p, VMX_F32, m->topw.as<float>(), m->topi.as<int32_t>(), T, E, k, 1, 0, stream)) return rc;
-            const bool few = pairs <= FP;   // every pair its own block: no sort
-            const int br = few ? 16 : (pairs >= 32 * E ? 64 : 16);
-            const int cap = few ? pairs * 16 : pairs + E * (br - 1);
-            const int32_t *fp = m->few_pairs.as<int32_t>();
-            const int32_t *up_rows = few ? fp : m->sorted.as<int32_t>(), *down_rows = few ? fp + FP * 16 : nullptr;
-            const int32_t *blk = few ? m->topi.as<int32_t>() : m->blk_expert.as<int32_t>();
-            const int32_t *total = few ? fp + 2 * FP * 16 + FP : m->total.as<int32_t>();
-            const int32_t *inv = few ? fp + 2 * FP * 16 : m->inv.as<int32_t>();
-            if (!few) {
-                if (int rc = vmx_moe_align_block_size(m->topi.as<int32_t>(), m->sorted.as<int32_t>(), m->blk_expert.as<int32_t>(),
-                                                      m->total.as<int32_t>(), pairs, E, br, cap, stream))
-                    return rc;
-                if (int rc = vmx_moe_inverse(m->inv.as<int32_t>(), m->sorted.as<int32_t>(), m->total.as<int32_t>(), pairs, cap, st)) return rc;
-            }
+            if (int rc = vmx_topk_softmax(m->rlogits.p, VMX_F32, b.topw.as<float>(), b.topi.as<int32_t>(), T, E, k, 1, 0, stream)) return rc;
+            if (int rc = b.plan(pairs, E, st)) return rc;
             VmxLinear u;   // gate | up of the pairs' rows in one product
             u.A = m->h.p, u.a_f32 = f32, u.lda = W;
             u.W = L.egu.as<uint16_t>(), u.w_sn = W, u.w_sk = 1;
             u.C = m->gu.p, u.c_f32 = 1, u.ldc = 2 * ff;
-            u.M = cap, u.N = 2 * ff, u.K = W, u.exact = f32;
-            u.row_ids = up_rows, u.row_div = k, u.row_limit = pairs;
-            u.block_expert = blk, u.expert_stride = (int64_t)2 * ff * W, u.block_rows = br, u.total_rows = total;
+            u.N = 2 * ff, u.K = W, u.exact = f32;
+            b.first(u, pairs, k, (int64_t)2 * ff * W);
             if (int rc = vmx_linear_launch(u, st)) return rc;
-            if (int rc = vmx_glu_silu_rows(m->act.p, f32, m->gu.as<float>(), cap, ff, st)) return rc;
+            if (int rc = vmx_glu_silu_rows(m->act.p, f32, m->gu.as<float>(), b.cap, ff, st)) return rc;
             VmxLinear d;
             d.A = m->act.p, d.a_f32 = f32, d.lda = ff;
             d.W = L.edown.as<uint16_t>(), d.w_sn = ff, d.w_sk = 1;
             d.C = m->ydown.p, d.c_f32 = 1, d.ldc = W;
-            d.M = cap, d.N = W, d.K = ff, d.exact = f32;
-            d.row_ids = down_rows, d.row_div = 1, d.row_limit = cap;
-            d.block_expert = blk, d.expert_stride = (int64_t)ff * W, d.block_rows = br, d.total_rows = total;
+            d.N = W, d.K = ff, d.exact = f32;
+            b.second(d, (int64_t)ff * W);
             if (int rc = vmx_linear_launch(d, st)) return rc;
-            if (int rc = vmx_moe_combine_f32(x, m->ydown.as<float>(), inv, m->topw.as<float>(), k, nullptr, fused + L.rg2_off, nf, T, W, st)) return rc;
+            if (int rc = vmx_moe_combine_f32(x, m->ydown.as<float>(), b.pair_rows, b.topw.as<float>(), k, nullptr, fused + L.rg2_off, nf, T, W, st)) return rc;
         }
         if (layer_trace)
             VMX_CHECK_HIP(hipMemcpyAsync(layer_trace + (size_t)li * T * W, x, (size_t)T * W * 4, hipMemcpyDeviceToDevice, st));

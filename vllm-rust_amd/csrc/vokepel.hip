@@ -16,34 +16,19 @@
 // by column offset.  The residual stream, norms, positions and angles, scores, softmax, the recurrence and its state are f32 in
 // both modes; VMX_BF16 rounds the operands of the linears and the cache rows to bf16, VMX_F32 multiplies in true f32 everywhere.
 // The forward call allocates nothing, reads nothing back and is graph-capturable.
-#include "vmx_kernels.h"
+#include "executor_common.h"
 #include <math.h>
-#include <algorithm>
-#include <string>
-#include <vector>
 
 namespace {
 
 using Buf = VmxBuf;
+using Seg = VmxTensorTable::Seg;
 
-int pad8(int n) { return (n + 7) & ~7; }
-
-struct Seg {       // where a checkpoint tensor lands: rows of the fused projection, or a buffer of its own
-    Buf *buf = nullptr;
-    size_t offset = 0, bytes = 0;
-};
-
-struct Layer {
+struct Layer : VmxTensorTable {
     vmx_vokepel_layer_config c;
     Buf norm1, norm2, wfused, bias, wo, wo_right, qnorm, knorm, r1, r2, talk, sink, inv_freq, wup, wdown;
     int nf = 0, q_off = 0, k_off = 0, v_off = 0, g_off = 0, z_off = 0, u_off = 0;
     int vdim = 0;   // value size of the attention as it runs (the talking attention's values are its keys)
-    std::vector<std::pair<std::string, Seg>> tensors;
-    std::vector<std::string> missing;
-    void want(const std::string &name, Buf *b, size_t off, size_t bytes) {
-        tensors.push_back({name, Seg{b, off, bytes}});
-        missing.push_back(name);
-    }
 };
 
 struct Run {       // one execution of a layer: its own cache and state
@@ -65,30 +50,6 @@ struct vmx_vokepel {
     size_t esz() const { return f32() ? 4 : 2; }
 };
 
-namespace {
-
-int upload(Buf &b, size_t offset, const void *data, size_t bytes, hipStream_t st) {
-    VMX_CHECK_HIP(hipMemcpyAsync((char *)b.p + offset, data, bytes, hipMemcpyDefault, st));
-    VMX_CHECK_HIP(hipStreamSynchronize(st));
-    return VMX_OK;
-}
-
-void erase_name(std::vector<std::string> &v, const std::string &n) {
-    for (size_t i = 0; i < v.size(); i++)
-        if (v[i] == n) {
-            v.erase(v.begin() + i);
-            return;
-        }
-}
-
-int alloc_zero(Buf &b, size_t n) {
-    if (int rc = b.alloc(n)) return rc;
-    VMX_CHECK_HIP(hipMemset(b.p, 0, n ? n : 16));
-    return VMX_OK;
-}
-
-}  // namespace
-
 extern "C" int vmx_vokepel_create(const vmx_vokepel_config *cfg, const vmx_vokepel_layer_config *layer_cfgs, vmx_vokepel **out) {
     VMX_REQUIRE(cfg && layer_cfgs && out, "vokepel_create: null pointer");
     const vmx_vokepel_config &c = *cfg;
@@ -106,9 +67,9 @@ extern "C" int vmx_vokepel_create(const vmx_vokepel_config *cfg, const vmx_vokep
     const size_t T = c.max_tokens, W = c.width, rows = (size_t)c.num_blocks * c.block_size;
     size_t attn_ws = 16, nf = 8, hv = 1, hd = 1, gw = 1, actn = 1;
     int rc = VMX_OK;
-#define GA(buf, n)                        \
-    do {                                  \
-        if (!rc) rc = alloc_zero(buf, n); \
+#define GA(buf, n)                            \
+    do {                                      \
+        if (!rc) rc = vmx_alloc_zero(buf, n); \
     } while (0)
 #define BAD(...)                    \
     {                               \
@@ -128,7 +89,7 @@ extern "C" int vmx_vokepel_create(const vmx_vokepel_config *cfg, const vmx_vokep
         int at = 0;
         auto seg = [&](int n) {
             const int o = at;
-            at = pad8(at + n);
+            at = vmx_pad8(at + n);
             return o;
         };
         L.want("norm1", &L.norm1, 0, W * 2);
@@ -310,8 +271,8 @@ extern "C" int vmx_vokepel_load_tensor(vmx_vokepel *m, const char *name, const v
     VMX_REQUIRE(dst.buf, "vokepel_load_tensor: unknown tensor `%s`", name);
     VMX_REQUIRE(bytes == dst.bytes, "vokepel_load_tensor: `%s`: expected %zu bytes of bf16, got %zu", name, dst.bytes, bytes);
     if (bytes > 0)
-        if (int rc = upload(*dst.buf, dst.offset, data, bytes, st)) return rc;
-    erase_name(*missing, key);
+        if (int rc = vmx_upload(*dst.buf, dst.offset, data, bytes, st)) return rc;
+    vmx_erase_name(*missing, key);
     return VMX_OK;
 }
 
