@@ -1027,6 +1027,90 @@ def gezozen_workload(prompt, steps, warmup, sizes=("1k", "2k"), batches=(1, 16),
             "prompt": prompt, "sizes": out}
 
 
+FOFINEX_SIZES = {
+    # name: (width, heads, dim, rot_dim, vdim, kv_rank, q_rank, memory heads, memory key / value size, dense ff, experts, top, groups, keep, expert_ff,
+    #        shared_ff, vocab)
+    "1k": (1024, 8, 64, 32, 64, 256, 384, 8, 128, 3072, 16, 4, 4, 2, 512, 512, 32000),
+    "2k": (2048, 16, 128, 64, 128, 512, 768, 16, 128, 6144, 32, 4, 4, 2, 1024, 1024, 32000),
+}
+
+
+def fofinex_workload(prompt, steps, warmup, sizes=("1k", "2k"), batches=(1, 16), comparator=True, main=True):
+    """Fofinex (sandwich layer norms; latent attention with latent queries and a shared cache beside a matrix memory with exponential
+    gates; biased GELU feed-forwards and corrected group-limited squared-ReLU experts with a gated shared expert; bf16 weights) at
+    layer sizes of real models, beside the closest existing models at equal size: Gesutar (latent attention + the same experts in every
+    layer) and, for the memory, Gezozen (the gated delta rule, with experts of the same width, in every layer).  Fofinex: attention +
+    dense, memory + experts, attention on the first layer's cache + dense, memory + experts.  Prompt pass: tokens/s of one
+    `prompt`-token sequence; decode: aggregate tok/s of B sequences at context `prompt`, one hipGraph per step.  main=False times the
+    comparators alone (kernel traces)."""
+    from vllm_rust_amd.fofinex import FofinexForCausalLM, FofinexLayerSpec, FofinexSpec, RotationSpec, synthetic_weights
+    from vllm_rust_amd.gesutar import GesutarForCausalLM, GesutarLayerSpec, GesutarSpec
+    from vllm_rust_amd.gesutar import synthetic_weights as gesutar_weights
+    from vllm_rust_amd.gezozen import GezozenForCausalLM, GezozenLayerSpec, GezozenSpec
+    from vllm_rust_amd.gezozen import synthetic_weights as gezozen_weights
+    out = {}
+    dev = torch.device("cuda", torch.cuda.current_device())
+    side = torch.cuda.Stream(device=dev)
+    BM = max(batches)
+    per_seq = (prompt + warmup + steps + 8 + 15) // 16 + 1
+
+    def timed(cls, spec, weights, V, recurrent):
+        model = cls(spec, "bfloat16", block_size=16, num_blocks=per_seq * BM, max_tokens=max(prompt, BM), max_seqs=BM)
+        model.load_state(weights(spec, 3, device=dev))
+        t = _packed_times(model, V, prompt, batches, warmup, steps, side, dev, recurrent)
+        model.close()
+        return t
+
+    def lines(t, macs, fixed, per_batch):
+        """macs: multiply-adds per prompt token; fixed: bytes a decode step reads whatever B; per_batch(B): the rest."""
+        r = {"prefill": {"tokens": prompt, "ms": round(t["prefill"] * 1e3, 3), "tok_s": round(prompt / t["prefill"], 1),
+                         "TFLOP_s": round(2.0 * prompt * macs / t["prefill"] / 1e12, 2)}}
+        for B in batches:
+            r[f"decode_b{B}"] = {"tok_s": round(B / t[B], 1), "ms_per_step": round(t[B] * 1e3, 4),
+                                 "GBps_algorithmic": round((fixed + per_batch(B)) / t[B] / 1e9, 1)}
+        return r
+    for name in sizes:
+        W, H, dim, rd, vd, R, Q, MH, MD, dff, E, top, G, keep, ff, sff, V = FOFINEX_SIZES[name]
+        sc = 1.0 / math.sqrt(dim + rd)
+        moe = dict(mlp="moe", experts=E, top=top, groups=G, keep_groups=keep, expert_ff=ff, shared_ff=sff)
+        att = dict(mixer="latent_attention", heads=H, dim=dim, rot_dim=rd, vdim=vd, kv_rank=R, q_rank=Q, scale=sc, mlp="dense", ff=dff,
+                   rot=RotationSpec(rd, 1e5, dict(factor=8.0, original=4096.0, fast=16.0, slow=2.0)))
+        mem = FofinexLayerSpec(mixer="mlstm", heads=MH, dim=MD, vdim=MD, gate_cap=15.0, router_scale=2.5, **moe)
+        spec = FofinexSpec(vocab=V, width=W, layers=[FofinexLayerSpec(**att), mem, FofinexLayerSpec(**att, kv_from=0), mem])
+        hv, md = H * vd, MH * MD
+        att_fl = H * (2 * R + rd) * prompt / 2                                            # MACs per token of one causal latent attention
+        experts = top * 2 * ff * W
+        rest = (E + 1 + 2 * sff) * W                                                      # router, shared expert
+        head = V * W / prompt
+        out[name] = {}
+        if main:
+            f_att = W * Q + Q * H * (dim + rd) + H * dim * R + hv * R + hv * W
+            lin = 2 * f_att + W * (R + rd) + 2 * 3 * dff * W + 2 * (W * (4 * md + 2 * MH) + md * W + rest)
+            t = timed(FofinexForCausalLM, spec, synthetic_weights, V, True)
+            out[name]["fofinex"] = lines(t, lin + 2 * experts + 2 * att_fl + 2 * MH * 3 * MD * MD + head, 2 * (lin + V * W),
+                                         lambda B: 2 * 2 * min(E, B * top) * 2 * ff * W + 2 * 2 * B * (prompt + 1) * (R + rd) + 2 * 2 * B * MH * MD * (MD + 1) * 4)
+        if comparator:
+            gl = GesutarLayerSpec(heads=H, dim=dim, rot_dim=rd, vdim=vd, kv_rank=R, window=8 * prompt, rot_dims=rd, rot_base=1e5, scale=sc, experts=E, top=top,
+                                  groups=G, keep_groups=keep, expert_ff=ff, shared_ff=sff, router_scale=1.0)
+            gs = GesutarSpec(vocab=V, width=W, layers=[gl] * 4, embed_scale=1.0, bigram_buckets=4093, bigram_mul_prev=31, bigram_mul_cur=7)
+            glin = 4 * (W * (H * (dim + rd) + R + rd + hv) + H * dim * R + hv * R + hv * W + rest)
+            t = timed(GesutarForCausalLM, gs, gesutar_weights, V, False)
+            out[name]["gesutar"] = lines(t, glin + 4 * experts + 4 * att_fl + head, 2 * (glin + V * W),
+                                         lambda B: 2 * 4 * min(E, B * top) * 2 * ff * W + 2 * 4 * B * (prompt + 1) * (R + rd))
+            zl = GezozenLayerSpec(mixer="delta", heads=MH, kv_heads=MH, dim=MD, vdim=MD, conv=4, mlp="moe", experts=E, top=top, expert_ff=ff, shared_ff=sff)
+            zs = GezozenSpec(vocab=V, width=W, layers=[zl] * 4, norm_groups=1, postln_alpha=2.0)
+            zlin = 4 * (W * (4 * md + 2 * MH) + md * W + 2 * W * W + (E + 1 + 3 * sff) * W)
+            t = timed(GezozenForCausalLM, zs, gezozen_weights, V, True)
+            out[name]["gezozen"] = lines(t, zlin + 4 * top * 3 * ff * W + 4 * MH * 3 * MD * MD + head, 2 * (zlin + V * W),
+                                         lambda B: 2 * 4 * min(E, B * top) * 3 * ff * W + 2 * 4 * B * MH * MD * MD * 4)
+        out[name]["config"] = {"width": W, "layers": ["latent_attention+dense", "mlstm+moe", "latent_attention(latents of layer 0)+dense", "mlstm+moe"],
+                               "heads": H, "dim": dim, "rot_dim": rd, "vdim": vd, "kv_rank": R, "q_rank": Q, "memory_heads": MH, "memory_dim": MD,
+                               "dense_ff": dff, "experts": E, "top": top, "groups": [G, keep], "expert_ff": ff, "shared_ff": sff, "vocab": V,
+                               "gesutar": ["latent_attention+moe"] * 4, "gezozen": ["delta+moe"] * 4}
+    return {"metric": "Fofinex prompt and decode throughput beside Gesutar and Gezozen at equal size", "unit": "tok/s", "dtype": "bf16",
+            "data": "synthetic", "prompt": prompt, "sizes": out}
+
+
 def plan_job(gpus, world, replicas_flag, weights, local_ranks):
     """What a launch of this script measures -- pure argument logic, no device.  N = 1: the single-GPU job.  N > 1 (one process
     per GPU under torch.distributed.run): ONE model tensor-parallel over the N ranks (BASELINE.json's metric is the TP curve at
@@ -1184,10 +1268,10 @@ def main():
     ap.add_argument("--no-secondary", action="store_true", help="skip the secondary measurements (other models at N = 1, replicas at N > 1)")
     ap.add_argument("--no-moe", action="store_true", help="skip the Mixtral-8x7B-shaped fused-MoE secondary measurement")
     ap.add_argument("--no-comparator", action="store_true",
-                    help="--workload vokepel / gezozen: time that executor alone (kernel traces of one model)")
-    ap.add_argument("--comparator-only", action="store_true", help="--workload gezozen: time the comparator alone (kernel traces of one model)")
-    ap.add_argument("--sizes", default="1k,2k", help="--workload vokepel / gezozen: which of its sizes to run")
-    ap.add_argument("--workload", choices=["all", "qwen3", "gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen"], default="all",
+                    help="--workload vokepel / gezozen / fofinex: time that executor alone (kernel traces of one model)")
+    ap.add_argument("--comparator-only", action="store_true", help="--workload gezozen / fofinex: time the comparators alone (kernel traces)")
+    ap.add_argument("--sizes", default="1k,2k", help="--workload vokepel / gezozen / fofinex: which of its sizes to run")
+    ap.add_argument("--workload", choices=["all", "qwen3", "gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen", "fofinex"], default="all",
                     help="profiling aid: run ONE workload alone (qwen3 = the primary without secondaries; the others print only "
                          "their own block), so that a kernel trace of the run holds that workload's launches only; gesutar = the Gesutar "
                          "executor (latent attention + grouped-router MoE, bf16) at two layer sizes beside the bf16 dense Qwen3 executor at "
@@ -1196,7 +1280,10 @@ def main():
                          "the same measurements; vokepel = the Vokepel executor (looped pre-norm layers, rotary sink attention beside a minimal "
                          "gated recurrent unit, mixed-head attention, bf16) at two layer sizes beside Gupuvik at equal size, the same measurements; "
                          "gezozen = the Gezozen executor (norm after the sum, attention beside gated linear attention / retention, per-head "
-                         "gated delta rule, sigmoid-routed experts, bf16) at two layer sizes beside Gupuvik at equal size, the same measurements")
+                         "gated delta rule, sigmoid-routed experts, bf16) at two layer sizes beside Gupuvik at equal size, the same measurements; "
+                         "fofinex = the Fofinex executor (sandwich layer norms, latent attention with latent queries, exponential-gate matrix "
+                         "memory, corrected group-limited experts, bf16) at two layer sizes beside Gesutar and Gezozen at equal size, the same "
+                         "measurements")
     ap.add_argument("--tp", action="store_true", help="accepted for compatibility: with --gpus N > 1 the tensor-parallel job is the default")
     ap.add_argument("--replicas", action="store_true",
                     help="with --gpus N > 1: N independent replicas as the primary (weak scaling, no collective) instead of ONE model "
@@ -1211,8 +1298,11 @@ def main():
     plan = plan_job(args.gpus, world, args.replicas, args.weights, d.local)
 
     K_steps, W_steps = args.steps, args.warmup
-    if args.workload in ("gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen"):   # one secondary alone (single GPU)
-        if args.workload == "gezozen":
+    if args.workload in ("gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen", "fofinex"):   # one secondary alone (single GPU)
+        if args.workload == "fofinex":
+            blk = fofinex_workload(max(args.prompt, 1024) if args.prompt == 256 else args.prompt, min(args.steps, 64), args.warmup,
+                                   sizes=tuple(args.sizes.split(",")), comparator=not args.no_comparator, main=not args.comparator_only)
+        elif args.workload == "gezozen":
             blk = gezozen_workload(max(args.prompt, 1024) if args.prompt == 256 else args.prompt, min(args.steps, 64), args.warmup,
                                    sizes=tuple(args.sizes.split(",")), comparator=not args.no_comparator, main=not args.comparator_only)
         elif args.workload == "vokepel":
