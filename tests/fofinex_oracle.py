@@ -10,11 +10,33 @@ heads with stretched rotation frequencies, a layer may read another layer's late
 input gate, forget gate, normaliser and running maximum).  Feed-forwards: biased tanh-GELU GLU; sigmoid-routed squared-ReLU experts
 chosen by corrected scores inside the best groups, plus a gated shared expert.
 """
+import contextlib
 import math
 
 import torch
 
 F = torch.float64
+_rounding = None        # None, or a function that rounds what enters a product
+
+
+@contextlib.contextmanager
+def rounded_operands(fn=lambda t: t.to(torch.bfloat16).to(F)):
+    """Inside, the activations that enter every linear map and what the latent cache keeps go through `fn` first: how far rounding
+    alone moves a model's results."""
+    global _rounding
+    _rounding = fn
+    try:
+        yield
+    finally:
+        _rounding = None
+
+
+def rnd(t):
+    return _rounding(t) if _rounding else t
+
+
+def lin(h, w):
+    return rnd(h) @ w.T
 
 
 # ------------------------------------------------------------------------------------------------ small pieces
@@ -85,29 +107,29 @@ def causal_softmax_attention(q, k, v, scale):
 def latents(h, w, pre, m, eps):
     """What a layer keeps per token: (normed latent [T, R], rotated key part [T, rot_dim])."""
     T, R = h.shape[0], m["kv_rank"]
-    y = h @ w[pre + "dkv"].T
+    y = lin(h, w[pre + "dkv"])
     c = rms_unit(y[:, :R], eps) * w[pre + "dkv.norm"]
-    return c, rotate(y[:, R:].unsqueeze(1), range(T), m.get("rot")).squeeze(1)
+    return rnd(c), rnd(rotate(y[:, R:].unsqueeze(1), range(T), m.get("rot")).squeeze(1))
 
 
 def latent_attention(h, w, pre, m, eps, kept):
     """kept: the (latent, rotated key part) this layer attends over, its own or another layer's."""
     T = h.shape[0]
     H, D, RD, V = m["heads"], m["dim"], m["rot_dim"], m["vdim"]
-    c_q = rms_unit(h @ w[pre + "dq"].T, eps) * w[pre + "dq.norm"]
-    q = (c_q @ w[pre + "uq"].T).reshape(T, H, D + RD)
-    q = torch.cat([q[:, :, :D], rotate(q[:, :, D:], range(T), m.get("rot"))], -1)
+    c_q = rms_unit(lin(h, w[pre + "dq"]), eps) * w[pre + "dq.norm"]
+    q = lin(c_q, w[pre + "uq"]).reshape(T, H, D + RD)
+    q = torch.cat([rnd(q[:, :, :D]), rotate(q[:, :, D:], range(T), m.get("rot"))], -1)
     c, k_rot = kept
     k = torch.cat([(c @ w[pre + "uk"].T).reshape(T, H, D), k_rot.unsqueeze(1).expand(T, H, RD)], -1)
     v = (c @ w[pre + "uv"].T).reshape(T, H, V)
-    return causal_softmax_attention(q, k, v, m["scale"]).reshape(T, H * V) @ w[pre + "o"].T
+    return lin(causal_softmax_attention(q, k, v, m["scale"]).reshape(T, H * V), w[pre + "o"])
 
 
 # ------------------------------------------------------------------------------------------------ matrix memory with exponential gates
-def exponential_gate_memory(q, k, v, log_i, log_f):
+def exponential_gate_memory(q, k, v, log_i, log_f, parts=None):
     """q, k [T, H, D], v [T, H, V], log_i, log_f [T, H].  Per head, from zero memory, zero normaliser and maximum 0:
     m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T;  n <- e^(f + m - m') n + e^(i - m') k;
-    o = S^T q / (max(|n . q|, e^(-m')) + 1e-6)."""
+    o = S^T q / (max(|n . q|, e^(-m')) + 1e-6).  parts (a list): receives (S^T q, n . q, e^(-m'), sum |n_i q_i|) per token."""
     T, H, D = q.shape
     S, n, m = torch.zeros(H, D, v.shape[2], dtype=F), torch.zeros(H, D, dtype=F), torch.zeros(H, dtype=F)
     out = []
@@ -117,8 +139,10 @@ def exponential_gate_memory(q, k, v, log_i, log_f):
         S = keep.reshape(H, 1, 1) * S + add.reshape(H, 1, 1) * k[t].unsqueeze(-1) * v[t].unsqueeze(-2)
         n = keep.reshape(H, 1) * n + add.reshape(H, 1) * k[t]
         m = m_new
-        down = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
-        out.append(torch.einsum("hdv,hd->hv", S, q[t]) / down.unsqueeze(-1))
+        top, nq = torch.einsum("hdv,hd->hv", S, q[t]), (n * q[t]).sum(-1)
+        out.append(top / (torch.maximum(nq.abs(), torch.exp(-m)) + 1e-6).unsqueeze(-1))
+        if parts is not None:
+            parts.append((top, nq, torch.exp(-m), (n * q[t]).abs().sum(-1)))
     return torch.stack(out)
 
 
@@ -129,22 +153,22 @@ def log_gates(zi, zf, cap):
 def mlstm(h, w, pre, m, eps):
     T = h.shape[0]
     H, D, V = m["heads"], m["dim"], m["vdim"]
-    q = (h @ w[pre + "q"].T).reshape(T, H, D) * D ** -0.5
-    k = (h @ w[pre + "k"].T).reshape(T, H, D)
-    v = (h @ w[pre + "v"].T).reshape(T, H, V)
-    li, lf = log_gates(h @ w[pre + "i"].T + w[pre + "i.b"], h @ w[pre + "f"].T + w[pre + "f.b"], m["gate_cap"])
+    q = (lin(h, w[pre + "q"])).reshape(T, H, D) * D ** -0.5
+    k = (lin(h, w[pre + "k"])).reshape(T, H, D)
+    v = (lin(h, w[pre + "v"])).reshape(T, H, V)
+    li, lf = log_gates(lin(h, w[pre + "i"]) + w[pre + "i.b"], lin(h, w[pre + "f"]) + w[pre + "f.b"], m["gate_cap"])
     o = rms_unit(exponential_gate_memory(q, k, v, li, lf), eps).reshape(T, H * V)
-    return (o * w[pre + "norm"] * torch.sigmoid(h @ w[pre + "g"].T)) @ w[pre + "o"].T
+    return lin(o * w[pre + "norm"] * torch.sigmoid(lin(h, w[pre + "g"])), w[pre + "o"])
 
 
 # ------------------------------------------------------------------------------------------------ feed-forward
 def dense_glu(h, w, pre):
-    g = gelu_tanh(h @ w[pre + "gate"].T + w[pre + "gate.b"])
-    return (g * (h @ w[pre + "up"].T + w[pre + "up.b"])) @ w[pre + "down"].T + w[pre + "down.b"]
+    g = gelu_tanh(lin(h, w[pre + "gate"]) + w[pre + "gate.b"])
+    return lin(g * (lin(h, w[pre + "up"]) + w[pre + "up.b"]), w[pre + "down"]) + w[pre + "down.b"]
 
 
 def expert(h, w, pre):
-    return relu_squared(h @ w[pre + "up"].T) @ w[pre + "down"].T
+    return lin(relu_squared(lin(h, w[pre + "up"])), w[pre + "down"])
 
 
 def choice_scores(z, correction, groups, keep):
@@ -185,7 +209,7 @@ def router_margin(z, correction, top, groups, keep):
 def mixture(h, w, pre, ff, margins=None):
     r = ff["router"]
     g = r.get("groups") or {"count": 1, "keep": 1}
-    z = h @ w[pre + "router"].T
+    z = lin(h, w[pre + "router"])
     ids, weight = route(z, w[pre + "correction"], r["top"], g["count"], g["keep"], r.get("scale", 1.0))
     if margins is not None:
         margins.append(router_margin(z, w[pre + "correction"], r["top"], g["count"], g["keep"]))
@@ -194,7 +218,7 @@ def mixture(h, w, pre, ff, margins=None):
         for e, s in zip(ids[t].tolist(), weight[t]):
             out[t] += s * expert(h[t:t + 1], w, f"{pre}e{e}.")[0]
     if ff.get("shared"):
-        out = out + expert(h, w, pre + "shared.") * torch.sigmoid(h @ w[pre + "shared.sg"].T)
+        out = out + expert(h, w, pre + "shared.") * torch.sigmoid(lin(h, w[pre + "shared.sg"]))
     return out
 
 
@@ -225,4 +249,4 @@ def forward(cfg, w, tokens, margins=None):
             y = feed_forward(layer_norm(x, w[pre + "norm2"], eps), w, pre + "mlp.", e["mlp"], margins)
             x = x + layer_norm(y, w[pre + "norm2b"], eps)
         trace.append(x)
-    return layer_norm(x, w["final.norm"], eps) @ w["embed"].T, torch.stack(trace)
+    return lin(layer_norm(x, w["final.norm"], eps), w["embed"]), torch.stack(trace)

@@ -4,7 +4,7 @@ normaliser fed in portions through dirty state slots, the read-out), then the ex
 different cuttings of the same tokens (whole prompts, token-by-token decoding, portions down to two tokens, unequal batches,
 recycled cache blocks and state slots), layers that share latents, norms of every row width, other sizes, random models, and greedy
 generation through the scheduler.  Small random models built here; float32 mode is held to 2e-4 of the logits' spread, bfloat16
-mode to 4e-2."""
+mode to 4e-2 or three times what rounding alone does."""
 import ctypes as C
 import dataclasses
 import json
@@ -86,14 +86,6 @@ def build(spec, dtype="float32", seed=0, tweak=None, block_size=4, num_blocks=96
     return model, Engine(model), {k: v.double() for k, v in ck.items()}
 
 
-def rel_err(got, want):
-    """Difference of two logits arrays, row means removed, relative to the spread of the expected rows (worst row)."""
-    g, w = np.asarray(got, np.float64), np.asarray(want, np.float64)
-    d = g - w
-    d = d - d.mean(-1, keepdims=True)
-    return float((np.sqrt((d ** 2).mean(-1)) / (w.std(-1) + 1e-12)).max())
-
-
 def tokens_for(spec, n, seed, weights=None, dtype="bfloat16"):
     """n random token ids.  With the model's weights: the first draw on which no router decision of the oracle is a close call
     (score gap above 0.01 for bfloat16 runs, 1e-5 for float32 ones), since a decision that rounding can flip says nothing about
@@ -109,6 +101,45 @@ def tokens_for(spec, n, seed, weights=None, dtype="bfloat16"):
         if not margins or min(margins) > gap:
             return toks
     raise AssertionError("no token draw with safe router margins")
+
+
+def row_errs(got, want):
+    """Difference of two logits arrays per row, row means removed, relative to the spread of the expected row."""
+    g, w = np.asarray(got, np.float64), np.asarray(want, np.float64)
+    d = g - w
+    d = d - d.mean(-1, keepdims=True)
+    return np.sqrt((d ** 2).mean(-1)) / (w.std(-1) + 1e-12)
+
+
+class Expected:
+    """The oracle's logits and streams of a token sequence, and how far a run may be from them: float32 2e-4 in every row; bfloat16
+    4e-2 in every row and 1.5e-2 in the mean, or three times what rounding the operands alone does to this model and these tokens
+    (a memory's read-out is divided by its own size, so some rows amplify rounding a lot)."""
+
+    def __init__(self, spec, weights, toks, dtype):
+        from tests import fofinex_oracle as orc
+        lg, tr = orc.forward(spec.to_config(), weights, toks)
+        self.logits, self.trace, self.dtype = lg.numpy(), tr.numpy(), dtype
+        self.rounded = None
+        if dtype == "bfloat16":
+            with orc.rounded_operands():
+                lg, tr = orc.forward(spec.to_config(), weights, toks)
+            self.rounded = (lg.numpy(), tr.numpy())
+
+    def _check(self, got, want, rounded, rows, what):
+        err = row_errs(got, want[rows])
+        if self.dtype == "float32":
+            assert err.max() < TOL["float32"], (what, err.max())
+            return
+        alone = row_errs(rounded, want)          # every row of the sequence: the worst one says what this model can amplify
+        assert err.max() < max(TOL["bfloat16"], 3 * alone.max()), (what, err.max(), alone.max())
+        assert len(err) < 8 or err.mean() < max(1.5e-2, 3 * alone.mean()), (what, err.mean(), alone.mean())
+
+    def check(self, got, rows=slice(None), what=""):
+        self._check(got, self.logits, self.rounded and self.rounded[0], rows, what)
+
+    def check_layer(self, i, got, what=""):
+        self._check(got, self.trace[i], self.rounded and self.rounded[1][i], slice(None), (what, "layer", i))
 
 
 def oracle(spec, weights, toks):
@@ -290,7 +321,7 @@ def test_causal_latent_attention_with_a_needle(gpu, H, R, rd, dtype, bs):
 
 def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul):
     """vmx_exp_gate_scan + vmx_matrix_memory_recurrence_ex over several sequences fed in unequal portions through slots that start
-    full of NaN.  Lists of [n, H, D], [n, H, D], [n, H, V], [n, H], [n, H]; returns o / (max(|n . q|, e^-m) + 1e-6) per sequence."""
+    full of NaN.  Lists of [n, H, D], [n, H, D], [n, H, V], [n, H], [n, H]; per sequence [o / (max(|n . q|, e^-m) + 1e-6), o, n . q, e^-m]."""
     from vllm_rust_amd._lib import MatrixMemoryOpts, check, lib
     H, D, V = k[0].shape[1], k[0].shape[2], v[0].shape[2]
     nslots = max(slot_of) + 2
@@ -324,13 +355,13 @@ def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul):
                                                   P.data_ptr(), S.data_ptr(), L.data_ptr(), len(slots), H, H, D, V, C.byref(mo), None))
         torch.cuda.synchronize()
         den = torch.maximum(norm[:, :H].abs(), floor[:, :H]).cpu().double() + 1e-6
-        res = o.cpu().double().reshape(T, H, V) / den.unsqueeze(-1)
+        res = [o.cpu().double().reshape(T, H, V) / den.unsqueeze(-1), o.cpu().double().reshape(T, H, V), norm[:, :H].cpu().double(), floor[:, :H].cpu().double()]
         row = 0
         for s, c in owners:
-            got[s].append(res[row:row + c])
+            got[s].append([r[row:row + c] for r in res])
             row += c
     assert fed == lens
-    return [torch.cat(x) for x in got]
+    return [[torch.cat([x[j] for x in g]) for j in range(4)] for g in got]
 
 
 @pytest.mark.parametrize("H,D,V,cap", [(2, 32, 32, 15.0), (3, 5, 7, 4.0), (4, 64, 47, 12.0), (1, 130, 16, 8.0), (2, 16, 1, 1.0), (5, 48, 64, 12.0)])
@@ -347,16 +378,21 @@ def test_exponential_memory_in_portions_through_dirty_slots(gpu, H, D, V, cap, b
     zi, zf = [(2 * rn(n, H) + bias[0]).float().double() for n in lens], [(2 * rn(n, H) + bias[1]).float().double() for n in lens]
     got = _run_exp_memory(torch, q, k, v, zi, zf, cap, [[90, 1, 1, 37, 2], [1], [2, 3, 63, 1, 1]], [3, 0, 4], D ** -0.5)
     for s in range(3):
-        want = orc.exponential_gate_memory(q[s] * D ** -0.5, k[s], v[s], *orc.log_gates(zi[s], zf[s], cap))
-        scale = max(1.0, float(want.abs().max()))
-        # where n . q nearly cancels, the quotient is as exact as that difference
-        assert float((got[s] - want).abs().max()) < 2e-4 * scale, s
+        parts = []
+        want = orc.exponential_gate_memory(q[s] * D ** -0.5, k[s], v[s], *orc.log_gates(zi[s], zf[s], cap), parts)
+        o, nq, floor, size = (torch.stack([p[j] for p in parts]) for j in range(4))
+        ref = max(1.0, float(size.max()))                          # the terms that o and n . q are sums of
+        assert float((got[s][1] - o).abs().max()) < 3e-5 * ref * max(1.0, float(v[s].abs().max())), s
+        assert float((got[s][2] - nq).abs().max()) < 2e-5 * ref, s
+        assert float((got[s][3] / floor - 1).abs().max()) < 3e-5, s
+        sound = (torch.maximum(nq.abs(), floor) > 0.05 * size).unsqueeze(-1)   # elsewhere the quotient is as exact as a cancellation
+        assert float(((got[s][0] - want) * sound).abs().max()) < 1e-3 * max(1.0, float((want * sound).abs().max())), s
 
 
 def test_exponential_memory_keeps_a_far_key_and_starts_at_zero(gpu):
     """A key written at position 5 with the largest input gate and asked for 290 tokens and four portions later, through a forget
     gate of nearly one on head 0 and of one half on head 1; before it the memory is empty of it.  The first token's floor is
-    e^-max(f, i): a maximum that started at minus infinity would give e^-i."""
+    e^-max(f, i), which leaves a small write small."""
     _, torch = gpu
     from tests import fofinex_oracle as orc
     n, D, V, cap = 300, 16, 8, 10.0
@@ -369,14 +405,14 @@ def test_exponential_memory_keeps_a_far_key_and_starts_at_zero(gpu):
     q[:, :, 0] = 1.0
     zi, zf = torch.full((n, 2), -4.0, dtype=torch.float64), torch.zeros(n, 2, dtype=torch.float64)
     zi[5], zf[:, 0] = 6.0, 90.0
-    got = _run_exp_memory(torch, [q], [k], [v], [zi], [zf], cap, [[4, 100, 1, 150, 45]], [1], 1.0)[0]
+    got = _run_exp_memory(torch, [q], [k], [v], [zi], [zf], cap, [[4, 100, 1, 150, 45]], [1], 1.0)[0][0]
     want = orc.exponential_gate_memory(q, k, v, *orc.log_gates(zi, zf, cap))
     assert float(got[:5].abs().max()) == 0 and float((got - want).abs().max()) < 1e-5
     for t in (5, 6, 104, 105, 295, 299):
         assert float((got[t, 0] - v[5, 0]).abs().max()) < 0.05 * float(v[5, 0].abs().max())      # still there, nearly whole
     assert float(got[40:, 1].abs().max()) < 1e-3 * float(v[5, 1].abs().max())
     k[0, :, 0] = 1.0                                                                               # the very first token, a small input gate
-    got = _run_exp_memory(torch, [q[:1]], [k[:1]], [v[:1]], [zi[:1]], [zf[:1]], cap, [[1]], [0], 1.0)[0]
+    got = _run_exp_memory(torch, [q[:1]], [k[:1]], [v[:1]], [zi[:1]], [zf[:1]], cap, [[1]], [0], 1.0)[0][0]
     m = torch.maximum(orc.log_gates(zi[0], zf[0], cap)[1], orc.log_gates(zi[0], zf[0], cap)[0])
     w = torch.exp(orc.log_gates(zi[0], zf[0], cap)[0])
     assert float((got[0] - v[0] * (w / torch.maximum(w, torch.ones(2, dtype=torch.float64))).unsqueeze(-1)).abs().max()) < 1e-5 and float(m[1]) < 0
@@ -415,11 +451,11 @@ def test_layers_and_logits_against_the_oracle(gpu, dtype):
     model, eng, w = build(spec, dtype)
     toks = tokens_for(spec, 41, 1, w, dtype)
     lg, _, tr = eng.step([("a", toks, list(range(len(toks))))], layer_trace=True)
-    want, wtr = oracle(spec, w, toks)
+    want = Expected(spec, w, toks, dtype)
     assert tr.shape[0] == len(spec.layers) == 5
     for r in range(tr.shape[0]):
-        assert rel_err(tr[r].cpu().numpy(), wtr[r]) < TOL[dtype], f"layer {r}"
-    assert rel_err(lg.cpu().numpy(), want) < TOL[dtype]
+        want.check_layer(r, tr[r].cpu().numpy())
+    want.check(lg.cpu().numpy())
 
 
 @pytest.mark.parametrize("kind", ["latent_attention", "mlstm"])
@@ -432,9 +468,9 @@ def test_every_layer_kind_alone(gpu, dtype, kind):
         model, eng, w = build(spec, dtype)
         toks = tokens_for(spec, 26, 2, w, dtype)
         lg, _, tr = eng.step([("a", toks, list(range(26)))], layer_trace=True)
-        want, wtr = oracle(spec, w, toks)
-        assert rel_err(tr[0].cpu().numpy(), wtr[0]) < TOL[dtype], (kind, ff)
-        assert rel_err(lg.cpu().numpy(), want) < TOL[dtype], (kind, ff)
+        want = Expected(spec, w, toks, dtype)
+        want.check_layer(0, tr[0].cpu().numpy())
+        want.check(lg.cpu().numpy(), what=(kind, ff))
         model.close()
 
 
@@ -443,10 +479,10 @@ def test_prompt_decode_and_portions_agree(gpu, dtype):
     spec = routed(small_spec(), dtype)
     model, eng, w = build(spec, dtype)
     toks = tokens_for(spec, 53, 2, w, dtype)
-    want, _ = oracle(spec, w, toks)
+    want = Expected(spec, w, toks, dtype)
     for cuts in ([53], [1], [2], [3], [7, 16], [16, 1], [20, 2, 1]):
         got = feed(eng, "s", toks, cuts)
-        assert rel_err(got, want) < TOL[dtype], f"cuts {cuts}"
+        want.check(got, what=f"cuts {cuts}")
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -458,7 +494,7 @@ def test_unequal_batches_and_recycled_blocks_and_slots(gpu, dtype):
     for gen in range(5):
         lens = [(29, 6), (3, 2), (14, 9)]
         reqs = {f"g{gen}r{i}": tokens_for(spec, n + d, 100 * gen + i, w, dtype) for i, (n, d) in enumerate(lens)}
-        want = {k: oracle(spec, w, t)[0] for k, t in reqs.items()}
+        want = {k: Expected(spec, w, t, dtype) for k, t in reqs.items()}
         got = {k: [] for k in reqs}
         lg, _, _ = eng.step([(k, reqs[k][:n], list(range(n))) for k, (n, _) in zip(reqs, lens)])
         at = 0
@@ -477,7 +513,7 @@ def test_unequal_batches_and_recycled_blocks_and_slots(gpu, dtype):
                 if fed[k] == len(reqs[k]):
                     eng.finish(k)     # leaves the batch early; its blocks and slot go back
         for k in reqs:
-            assert rel_err(np.concatenate(got[k]), want[k]) < TOL[dtype], k
+            want[k].check(np.concatenate(got[k]), what=k)
     assert len(eng.blocks.free) == 40 and len(eng.states.free) == 3
 
 
@@ -497,7 +533,7 @@ def test_mixed_steps_of_portions_and_decoding(gpu, dtype):
             at, fed[k] = at + n, fed[k] + n
     for k in reqs:
         assert fed[k] == len(reqs[k])
-        assert rel_err(np.concatenate(got[k]), oracle(spec, w, reqs[k])[0]) < TOL[dtype], k
+        Expected(spec, w, reqs[k], dtype).check(np.concatenate(got[k]), what=k)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -510,11 +546,11 @@ def test_layers_that_share_latents(gpu, dtype):
     spec = small_spec(layers=layers)
     model, eng, w = build(spec, dtype)
     toks = tokens_for(spec, 45, 7)
-    want, wtr = oracle(spec, w, toks)
+    want = Expected(spec, w, toks, dtype)
     other = dataclasses.replace(spec, layers=[dataclasses.replace(l, kv_from=2) if l.kv_from == 0 else l for l in layers])
-    assert rel_err(oracle(other, w, toks)[0], want) > 0.2
+    assert row_errs(oracle(other, w, toks)[0], want.logits).mean() > 0.2
     for cuts in ([45], [20, 1], [2]):
-        assert rel_err(feed(eng, "a", toks, cuts), want) < TOL[dtype]
+        want.check(feed(eng, "a", toks, cuts))
     model.close()
     from vllm_rust_amd._lib import VmxError
     from vllm_rust_amd.fofinex import FofinexForCausalLM
@@ -535,11 +571,11 @@ def test_norms_of_every_row_width(gpu, dtype, width):
     spec = sure_routing(small_spec(layers=[att_layer(heads=2), mem_layer(heads=2, experts=3, groups=1, keep_groups=1)], width=width, vocab=31))
     model, eng, w = build(spec, dtype, tweak=offset, max_tokens=32, num_blocks=16)
     toks = tokens_for(spec, 9, width)
-    want, wtr = oracle(spec, w, toks)
+    want = Expected(spec, w, toks, dtype)
     lg, _, tr = eng.step([("a", toks, list(range(9)))], layer_trace=True)
     if width > 1:
-        assert rel_err(tr[-1].cpu().numpy(), wtr[-1]) < TOL[dtype]
-        assert rel_err(lg.cpu().numpy(), want) < TOL[dtype]
+        want.check_layer(-1, tr[-1].cpu().numpy())
+        want.check(lg.cpu().numpy())
     else:
         assert float(tr.abs().max()) == 0 and float(lg.abs().max()) == 0          # one number minus itself
     model.close()
@@ -552,9 +588,9 @@ def test_large_eps_shows_the_scales_that_norms_hide(gpu, dtype):
     spec = routed(small_spec(layers=[mem_layer(mlp=None), att_layer(mlp=None), mem_layer(heads=2, dim=40, **DENSE)], norm_eps=0.5), dtype)
     model, eng, w = build(spec, dtype)
     toks = tokens_for(spec, 48, 3, w, dtype)
-    want, _ = oracle(spec, w, toks)
+    want = Expected(spec, w, toks, dtype)
     for cuts in ([48], [20, 1]):
-        assert rel_err(feed(eng, "a", toks, cuts), want) < TOL[dtype]
+        want.check(feed(eng, "a", toks, cuts))
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -576,9 +612,9 @@ def test_sharp_attention_over_300_tokens_and_long_decoding(gpu, dtype, sizes):
     spec = sure_routing(small_spec(layers=layers))
     model, eng, w = build(spec, dtype, tweak=sharpen, block_size=16, num_blocks=64, max_tokens=512)
     toks = tokens_for(spec, 300, 9)
-    want, _ = oracle(spec, w, toks)
-    assert rel_err(feed(eng, "a", toks, [220, 1]), want) < TOL[dtype]
-    assert rel_err(feed(eng, "b", toks, [300]), want) < TOL[dtype]
+    want = Expected(spec, w, toks, dtype)
+    want.check(feed(eng, "a", toks, [220, 1]))
+    want.check(feed(eng, "b", toks, [300]))
 
 
 OTHER_SIZES = {
@@ -614,14 +650,14 @@ def test_other_sizes(gpu, dtype, name):
     spec = routed(small_spec(**kw), dtype)
     model, eng, w = build(spec, dtype)
     toks = tokens_for(spec, 37, 4, w, dtype)
-    want, wtr = oracle(spec, w, toks)
+    want = Expected(spec, w, toks, dtype)
     lg, _, tr = eng.step([("a", toks, list(range(37)))], layer_trace=True)
     assert tr.shape[0] == len(spec.layers)
-    assert rel_err(tr[-1].cpu().numpy(), wtr[-1]) < TOL[dtype]
-    assert rel_err(lg.cpu().numpy(), want) < TOL[dtype]
+    want.check_layer(-1, tr[-1].cpu().numpy())
+    want.check(lg.cpu().numpy())
     eng.finish("a")
-    assert rel_err(feed(eng, "b", toks, [30, 1]), want) < TOL[dtype]
-    assert rel_err(feed(eng, "c", toks, [2]), want) < TOL[dtype]
+    want.check(feed(eng, "b", toks, [30, 1]))
+    want.check(feed(eng, "c", toks, [2]))
 
 
 def random_spec(rng):
@@ -666,7 +702,7 @@ def test_random_models(gpu, dtype, seed):
     bs = int(rng.choice([1, 3, 4, 8, 16]))
     model, eng, w = build(spec, dtype, seed=seed, block_size=bs, num_blocks=600 // bs + 8)
     ta, tb, tc = tokens_for(spec, 75, seed, w, dtype), tokens_for(spec, 33, seed + 50, w, dtype), tokens_for(spec, 60, seed + 99, w, dtype)
-    wa, wb, wc = (oracle(spec, w, t)[0] for t in (ta, tb, tc))
+    wa, wb, wc = (Expected(spec, w, t, dtype) for t in (ta, tb, tc))
     lg, _, _ = eng.step([("a", ta[:60], list(range(60))), ("b", tb[:20], list(range(20)))])
     ga, gb = [lg[:60].cpu().numpy()], [lg[60:].cpu().numpy()]
     for i in range(15):
@@ -677,9 +713,9 @@ def test_random_models(gpu, dtype, seed):
             gb.append(lg[1:2].cpu().numpy())
         if i == 12:
             eng.finish("b")
-    assert rel_err(np.concatenate(ga), wa) < TOL[dtype]
-    assert rel_err(np.concatenate(gb), wb) < TOL[dtype]
-    assert rel_err(feed(eng, "c", tc, [int(rng.integers(2, 20)), int(rng.integers(1, 9))]), wc) < TOL[dtype]
+    wa.check(np.concatenate(ga))
+    wb.check(np.concatenate(gb))
+    wc.check(feed(eng, "c", tc, [int(rng.integers(2, 20)), int(rng.integers(1, 9))]))
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -779,9 +815,11 @@ def test_registry_and_command_line_tools(gpu, tmp_path):
     model = load_model(d, dtype="float32", max_tokens=128, max_seqs=4, block_size=8)
     assert model.spec.to_config() == spec.to_config()
     ta, tb = tokens_for(spec, 30, 1), tokens_for(spec, 12, 2)
-    wa, wb = oracle(spec, w, ta)[0], oracle(spec, w, tb)[0]
+    wa, wb = {}, {}
+    for dt in TOL:
+        wa[dt], wb[dt] = Expected(spec, w, ta, dt), Expected(spec, w, tb, dt)
     lg, _, _ = Engine(model).step([("x", ta, [29])])
-    assert rel_err(lg.cpu().numpy(), wa[29:30]) < TOL["float32"]
+    wa["float32"].check(lg.cpu().numpy(), [29])
     model.close()
     steps = [{"step": 0, "entries": [{"id": "a", "tokens": ta[:20], "want": [0, 19]}, {"id": "b", "tokens": tb[:10], "want": [9]}], "end": []},
              {"step": 1, "entries": [{"id": "a", "tokens": [ta[20]], "want": [0]}, {"id": "b", "tokens": [tb[10]], "want": []}], "end": []},
@@ -794,10 +832,12 @@ def test_registry_and_command_line_tools(gpu, tmp_path):
         assert r.returncode == 0, r.stderr
         assert [l for l in r.stdout.splitlines() if l.startswith("done")] == [f"done {i}" for i in range(4)]
         rd = lambda i: np.fromfile(out / f"{i}.f32", dtype="<f4").reshape(-1, spec.vocab)   # noqa: E731
-        assert rel_err(rd(0), np.stack([wa[0], wa[19], wb[9]])) < TOL[dtype]
-        assert rel_err(rd(1), wa[20:21]) < TOL[dtype]
-        assert rel_err(rd(2), np.stack([wa[21], wb[11]])) < TOL[dtype]
-        assert rel_err(rd(3), wa[29:30]) < TOL[dtype]
+        wa[dtype].check(rd(0)[:2], [0, 19])
+        wb[dtype].check(rd(0)[2:], [9])
+        wa[dtype].check(rd(1), [20])
+        wa[dtype].check(rd(2)[:1], [21])
+        wb[dtype].check(rd(2)[1:], [11])
+        wa[dtype].check(rd(3), [29])
     r = subprocess.run([sys.executable, str(ROOT / "bin" / "generate"), "--model", str(d), "--dtype", "float32", "--prompt", ",".join(map(str, ta[:9])),
                         "--max-new-tokens", "4"], capture_output=True, text=True, timeout=300)
     assert r.returncode == 0, r.stderr
