@@ -23,7 +23,7 @@
 // Exponential gates (vmx_exp_gate_scan): a memory whose input gate is an exponential keeps the logarithm of its scale, a running
 // maximum m_t = max(f_t + m_(t-1), i_t) per head (from 0), in its slot; what the recurrence needs are the decay
 // exp(f_t + m_(t-1) - m_t), the write gain exp(i_t - m_t) and, for the read-out, exp(-m_t).  The maximum is a prefix scan over
-// (sum of f, largest of "i plus the f after it") pairs: one wave per (sequence, head), 64 tokens a round.
+// (sum of f, largest of "i plus the f after it") pairs: one workgroup per (sequence, head), 256 tokens a round.
 #include "vmx_kernels.h"
 
 namespace {
@@ -269,23 +269,26 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(const DeltaArgs a
     for (int u = 0; u < DPT; u++) sp[(int64_t)u * 256] = S[u];
 }
 
-// In place, one wave per (sequence, head): i[t, h] <- exp(i_t - m_t), f[t, h] <- exp(f_t + m_(t-1) - m_t), floor[t, h] = exp(-m_t)
+// In place, one workgroup per (sequence, head): i[t, h] <- exp(i_t - m_t), f[t, h] <- exp(f_t + m_(t-1) - m_t), floor[t, h] = exp(-m_t)
 // with i_t = cap tanh(i / cap), f_t = log(sigmoid(cap tanh(f / cap))) and m the running maximum (the slot's; 0 at position 0).
-__global__ __launch_bounds__(64) void exp_gate_scan_kernel(float *__restrict__ ig, int64_t ldi, float *__restrict__ fg, int64_t ldf,
-                                                            float *__restrict__ floor, int64_t ldfloor, float *__restrict__ m_state, float cap,
-                                                            const int32_t *__restrict__ positions, const int32_t *__restrict__ seq_starts,
-                                                            const int32_t *__restrict__ state_slots, int heads) {
-    const int h = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x;
+__global__ __launch_bounds__(256) void exp_gate_scan_kernel(float *__restrict__ ig, int64_t ldi, float *__restrict__ fg, int64_t ldf,
+                                                             float *__restrict__ floor, int64_t ldfloor, float *__restrict__ m_state, float cap,
+                                                             const int32_t *__restrict__ positions, const int32_t *__restrict__ seq_starts,
+                                                             const int32_t *__restrict__ state_slots, int heads) {
+    __shared__ float tot[2][4][2];     // the waves' totals of a round, double-buffered
+    const int h = blockIdx.x, seq = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int first = seq_starts[seq], count = seq_starts[seq + 1] - first;
     if (count <= 0) return;
     float *ms = m_state + (int64_t)state_slots[seq] * heads + h;
     float m0 = positions[first] == 0 ? 0.f : *ms;
-    for (int t0 = 0; t0 < count; t0 += 64) {
-        const bool in = t0 + lane < count;
-        const int64_t row = first + t0 + lane;
-        const float li = in ? cap * tanhf(ig[row * ldi + h] / cap) : -1e30f;
-        const float lf = in ? -softplus_f(-cap * tanhf(fg[row * ldf + h] / cap)) : 0.f;
-        float A = lf, B = li;      // over the tokens of this round up to this lane's: sum of f; largest i plus the f after it
+    float zi = tid < count ? ig[(int64_t)(first + tid) * ldi + h] : 0.f, zf = tid < count ? fg[(int64_t)(first + tid) * ldf + h] : 0.f;
+    for (int t0 = 0, b = 0; t0 < count; t0 += 256, b ^= 1) {
+        const bool in = t0 + tid < count;
+        const int64_t row = first + t0 + tid;
+        const float li = in ? cap * tanhf(zi / cap) : -1e30f;
+        const float lf = in ? -softplus_f(-cap * tanhf(zf / cap)) : 0.f;
+        if (t0 + 256 + tid < count) zi = ig[(row + 256) * ldi + h], zf = fg[(row + 256) * ldf + h];   // the next round's, while this one is scanned
+        float A = lf, B = li;      // over the wave's tokens up to this lane's: sum of f; largest i plus the f after it
 #pragma unroll
         for (int d = 1; d < 64; d <<= 1) {
             const float pa = __shfl_up(A, d, 64), pb = __shfl_up(B, d, 64);
@@ -294,15 +297,23 @@ __global__ __launch_bounds__(64) void exp_gate_scan_kernel(float *__restrict__ i
                 A += pa;
             }
         }
-        const float m = fmaxf(m0 + A, B), up = __shfl_up(m, 1, 64), prev = lane == 0 ? m0 : up;
+        if (lane == 63) tot[b][wave][0] = A, tot[b][wave][1] = B;
+        __syncthreads();
+        float before = m0, end = m0;   // the maximum ahead of this wave's first token, and after the round
+#pragma unroll
+        for (int w = 0; w < 4; w++) {
+            if (w == wave) before = end;
+            end = fmaxf(end + tot[b][w][0], tot[b][w][1]);
+        }
+        const float m = fmaxf(before + A, B), up = __shfl_up(m, 1, 64), prev = lane == 0 ? before : up;
         if (in) {
             ig[row * ldi + h] = expf(li - m);
             fg[row * ldf + h] = expf(lf + prev - m);
             floor[row * ldfloor + h] = expf(-m);
         }
-        m0 = __shfl(m, min(63, count - t0 - 1), 64);
+        m0 = end;
     }
-    if (lane == 0) *ms = m0;
+    if (tid == 0) *ms = m0;
 }
 
 // y[t, h] = o[t, h] / sqrt(mean(o^2) + eps) * w * sigmoid(gate[t, h]) (gate_silu: * silu(gate[t, h])); one wave per (token, head);
@@ -485,7 +496,7 @@ extern "C" int vmx_exp_gate_scan(float *input_gate, int64_t ldi, float *forget_g
     VMX_REQUIRE(input_gate && forget_gate && floor && max_state && positions && seq_starts && state_slots, "exp_gate_scan: null pointer");
     VMX_REQUIRE(heads >= 1 && ldi >= heads && ldf >= heads && ldfloor >= heads && cap > 0.f, "exp_gate_scan: bad sizes or cap");
     if (num_seqs <= 0) return VMX_OK;
-    hipLaunchKernelGGL(exp_gate_scan_kernel, dim3(heads, num_seqs), dim3(64), 0, vmx_stream(stream), input_gate, ldi, forget_gate, ldf, floor, ldfloor,
+    hipLaunchKernelGGL(exp_gate_scan_kernel, dim3(heads, num_seqs), dim3(256), 0, vmx_stream(stream), input_gate, ldi, forget_gate, ldf, floor, ldfloor,
                        max_state, cap, positions, seq_starts, state_slots, heads);
     VMX_CHECK_LAUNCH("exp_gate_scan");
     return VMX_OK;

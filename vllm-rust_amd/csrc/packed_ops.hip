@@ -72,88 +72,176 @@ __global__ __launch_bounds__(256) void row_norm_f32in_kernel(void *__restrict__ 
 
 // Both norms around a residual sum in one pass over the row: x <- [x +] N(y) * w_post, h = N(x) * w_next (w_next NULL: no h).
 // y[t] is a row of numbers, a row of the embedding table, or the combined result of a mixture of experts.  N as above, centred or
-// not.  HELD > 0: a thread keeps its HELD numbers of the row in registers from the first read to the last store; 0: any width, y
-// is formed anew in every pass (at most three) and the new x is read back by the thread that wrote it.
-template <int HELD>
+// not.  A thread keeps HELD groups of VEC neighbouring columns in registers from the first read to the last store, and every load
+// that does not depend on a statistic is issued before the first one.  HELD 0: any width, y is formed anew in every pass (at most
+// three) and the new x is read back by the thread that wrote it.
+template <int VEC> struct SandwichVec;
+template <> struct SandwichVec<4> {
+    static __device__ __forceinline__ void ld(const float *p, float *v) {
+        const float4 f = *reinterpret_cast<const float4 *>(p);
+        v[0] = f.x, v[1] = f.y, v[2] = f.z, v[3] = f.w;
+    }
+    static __device__ __forceinline__ void ld(const uint16_t *p, float *v) {
+        const uint2 u = *reinterpret_cast<const uint2 *>(p);
+        v[0] = vmx_bf16_to_f32((uint16_t)u.x), v[1] = vmx_bf16_to_f32((uint16_t)(u.x >> 16));
+        v[2] = vmx_bf16_to_f32((uint16_t)u.y), v[3] = vmx_bf16_to_f32((uint16_t)(u.y >> 16));
+    }
+    static __device__ __forceinline__ void st(float *p, const float *v) { *reinterpret_cast<float4 *>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+    static __device__ __forceinline__ void st(uint16_t *p, const float *v) {
+        *reinterpret_cast<uint2 *>(p) = make_uint2((uint32_t)vmx_f32_to_bf16(v[0]) | ((uint32_t)vmx_f32_to_bf16(v[1]) << 16),
+                                                   (uint32_t)vmx_f32_to_bf16(v[2]) | ((uint32_t)vmx_f32_to_bf16(v[3]) << 16));
+    }
+};
+template <> struct SandwichVec<1> {
+    static __device__ __forceinline__ void ld(const float *p, float *v) { v[0] = p[0]; }
+    static __device__ __forceinline__ void ld(const uint16_t *p, float *v) { v[0] = vmx_bf16_to_f32(p[0]); }
+    static __device__ __forceinline__ void st(float *p, const float *v) { p[0] = v[0]; }
+    static __device__ __forceinline__ void st(uint16_t *p, const float *v) { p[0] = vmx_f32_to_bf16(v[0]); }
+};
+
+template <int HELD, int VEC>
 __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a) {
-    __shared__ float red[4];
-    constexpr int PT = HELD ? HELD : 1;
-    const int t = blockIdx.x, W = a.width;
+    using V = SandwichVec<VEC>;
+    __shared__ float red[4][4];      // a row per reduction: one barrier each
+    constexpr int G = HELD ? HELD : 1;
+    const int t = blockIdx.x, tid = threadIdx.x, W = a.width;
     float *x = a.x + (int64_t)t * W;
     const float inv_w = 1.0f / (float)W;
-    int64_t erow = 0;
+    auto block_sum = [&](float v, int k) {
+        v = vmx_wave_sum(v);
+        if ((tid & 63) == 0) red[k][tid >> 6] = v;
+        __syncthreads();
+        return (red[k][0] + red[k][1]) + (red[k][2] + red[k][3]);
+    };
+    const float sg = a.shared_gate ? 1.0f / (1.0f + expf(-a.shared_gate[(int64_t)t * a.ld_shared_gate])) : 1.0f;
+    const uint16_t *erow = nullptr;
     if (a.embed) {
         const int id = a.tokens[t];
-        erow = (int64_t)(id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id)) * W;
+        erow = a.embed + (int64_t)(id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id)) * W;
     }
-    const float sg = a.shared_gate ? 1.0f / (1.0f + expf(-a.shared_gate[(int64_t)t * a.ld_shared_gate])) : 1.0f;
-    auto y_at = [&](int i) {
-        if (a.embed) return vmx_bf16_to_f32(a.embed[erow + i]);
-        if (!a.pair_rows) return a.y[(int64_t)t * W + i];
-        float v = 0.f;
-        for (int s = 0; s < a.top; s++) v = fmaf(a.pair_w[(int64_t)t * a.top + s], a.y[(int64_t)a.pair_rows[(int64_t)t * a.top + s] * W + i], v);
-        if (a.shared) v = fmaf(sg, a.shared[(int64_t)t * W + i], v);
-        return v;
-    };
-    // sum of f over the row's columns, in the same order for every HELD
-    float held[PT];
-    auto over_row = [&](auto &&f) {
-        float s = 0.f;
-        if constexpr (HELD > 0) {
-#pragma unroll
-            for (int u = 0; u < PT; u++)
-                if (threadIdx.x + 256 * u < W) s += f(threadIdx.x + 256 * u, u);
-        } else {
-            for (int i = threadIdx.x; i < W; i += 256) s += f(i, 0);
-        }
-        return vmx_block_sum_256(s, red);
-    };
-    auto norm_of = [&](auto &&at, float &mean) {   // at(i, u): the row; returns 1 / sqrt(statistic + eps)
-        mean = a.centered ? over_row(at) * inv_w : 0.f;
-        const float ss = over_row([&](int i, int u) {
-            const float d = at(i, u) - mean;
-            return d * d;
-        });
-        return 1.0f / sqrtf(ss * inv_w + a.eps);
-    };
     if constexpr (HELD > 0) {
+        float y[G][VEC], xv[G][VEC], wp[G][VEC], wn[G][VEC];
+        int col[G];
+        bool in[G];
 #pragma unroll
-        for (int u = 0; u < PT; u++) {
-            const int i = threadIdx.x + 256 * u;
-            held[u] = i < W ? y_at(i) : 0.f;
+        for (int u = 0; u < G; u++) {
+            col[u] = VEC * (tid + 256 * u);
+            in[u] = col[u] < W;
+#pragma unroll
+            for (int e = 0; e < VEC; e++) y[u][e] = xv[u][e] = wp[u][e] = wn[u][e] = 0.f;
         }
-    }
-    float mean;
-    float inv = norm_of([&](int i, int u) { return HELD ? held[u] : y_at(i); }, mean);
-    auto update = [&](int i, float y) {
-        const float v = (a.accumulate ? x[i] : 0.f) + (y - mean) * inv * vmx_bf16_to_f32(a.w_post[i]);
-        x[i] = v;
-        return v;
-    };
-    if constexpr (HELD > 0) {
 #pragma unroll
-        for (int u = 0; u < PT; u++) {
-            const int i = threadIdx.x + 256 * u;
-            if (i < W) held[u] = update(i, held[u]);
+        for (int u = 0; u < G; u++)
+            if (in[u]) {
+                if (a.embed) V::ld(erow + col[u], y[u]);
+                else if (!a.pair_rows) V::ld(a.y + (int64_t)t * W + col[u], y[u]);
+                if (a.accumulate) V::ld(x + col[u], xv[u]);
+                V::ld(a.w_post + col[u], wp[u]);
+                if (a.w_next) V::ld(a.w_next + col[u], wn[u]);
+            }
+        if (a.pair_rows && !a.embed) {
+            for (int s0 = 0; s0 < a.top; s0 += 4) {     // four experts' rows in flight
+                float w4[4];
+                int64_t r4[4];
+#pragma unroll
+                for (int s = 0; s < 4; s++) {
+                    const int64_t p = (int64_t)t * a.top + min(s0 + s, a.top - 1);
+                    w4[s] = s0 + s < a.top ? a.pair_w[p] : 0.f;
+                    r4[s] = (int64_t)a.pair_rows[p] * W;
+                }
+#pragma unroll
+                for (int u = 0; u < G; u++)
+                    if (in[u]) {
+                        float v[4][VEC];
+#pragma unroll
+                        for (int s = 0; s < 4; s++) V::ld(a.y + r4[s] + col[u], v[s]);
+#pragma unroll
+                        for (int s = 0; s < 4; s++)
+#pragma unroll
+                            for (int e = 0; e < VEC; e++) y[u][e] = fmaf(w4[s], v[s][e], y[u][e]);
+                    }
+            }
+            if (a.shared)
+#pragma unroll
+                for (int u = 0; u < G; u++)
+                    if (in[u]) {
+                        float v[VEC];
+                        V::ld(a.shared + (int64_t)t * W + col[u], v);
+#pragma unroll
+                        for (int e = 0; e < VEC; e++) y[u][e] = fmaf(sg, v[e], y[u][e]);
+                    }
+        }
+        auto statistics = [&](const float (&v)[G][VEC], int k, float &mean) {
+            mean = 0.f;
+            if (a.centered) {
+                float s = 0.f;
+#pragma unroll
+                for (int u = 0; u < G; u++)
+#pragma unroll
+                    for (int e = 0; e < VEC; e++) s += v[u][e];     // columns past the row are 0
+                mean = block_sum(s, k) * inv_w;
+            }
+            float ss = 0.f;
+#pragma unroll
+            for (int u = 0; u < G; u++)
+#pragma unroll
+                for (int e = 0; e < VEC; e++) {
+                    const float d = in[u] ? v[u][e] - mean : 0.f;
+                    ss = fmaf(d, d, ss);
+                }
+            return 1.0f / sqrtf(block_sum(ss, k + 1) * inv_w + a.eps);
+        };
+        float mean;
+        float inv = statistics(y, 0, mean);
+#pragma unroll
+        for (int u = 0; u < G; u++) {
+#pragma unroll
+            for (int e = 0; e < VEC; e++) xv[u][e] = in[u] ? xv[u][e] + (y[u][e] - mean) * inv * wp[u][e] : 0.f;
+            if (in[u]) V::st(x + col[u], xv[u]);
+        }
+        if (!a.w_next) return;
+        inv = statistics(xv, 2, mean);
+#pragma unroll
+        for (int u = 0; u < G; u++) {
+            if (!in[u]) continue;
+#pragma unroll
+            for (int e = 0; e < VEC; e++) xv[u][e] = (xv[u][e] - mean) * inv * wn[u][e];
+            if (a.h_f32) V::st((float *)a.h + (int64_t)t * W + col[u], xv[u]);
+            else V::st((uint16_t *)a.h + (int64_t)t * W + col[u], xv[u]);
         }
     } else {
-        for (int i = threadIdx.x; i < W; i += 256) update(i, y_at(i));
-    }
-    if (!a.w_next) return;
-    inv = norm_of([&](int i, int u) { return HELD ? held[u] : x[i]; }, mean);
-    auto store = [&](int i, float v) {
-        v = (v - mean) * inv * vmx_bf16_to_f32(a.w_next[i]);
-        if (a.h_f32) ((float *)a.h)[(int64_t)t * W + i] = v;
-        else ((uint16_t *)a.h)[(int64_t)t * W + i] = vmx_f32_to_bf16(v);
-    };
-    if constexpr (HELD > 0) {
-#pragma unroll
-        for (int u = 0; u < PT; u++) {
-            const int i = threadIdx.x + 256 * u;
-            if (i < W) store(i, held[u]);
+        auto y_at = [&](int i) {
+            if (a.embed) return vmx_bf16_to_f32(erow[i]);
+            if (!a.pair_rows) return a.y[(int64_t)t * W + i];
+            float v = 0.f;
+            for (int s = 0; s < a.top; s++) v = fmaf(a.pair_w[(int64_t)t * a.top + s], a.y[(int64_t)a.pair_rows[(int64_t)t * a.top + s] * W + i], v);
+            if (a.shared) v = fmaf(sg, a.shared[(int64_t)t * W + i], v);
+            return v;
+        };
+        auto statistics = [&](auto &&at, int k, float &mean) {
+            mean = 0.f;
+            if (a.centered) {
+                float s = 0.f;
+                for (int i = tid; i < W; i += 256) s += at(i);
+                mean = block_sum(s, k) * inv_w;
+            }
+            float ss = 0.f;
+            for (int i = tid; i < W; i += 256) {
+                const float d = at(i) - mean;
+                ss = fmaf(d, d, ss);
+            }
+            return 1.0f / sqrtf(block_sum(ss, k + 1) * inv_w + a.eps);
+        };
+        float mean;
+        float inv = statistics(y_at, 0, mean);
+        for (int i = tid; i < W; i += 256) x[i] = (a.accumulate ? x[i] : 0.f) + (y_at(i) - mean) * inv * vmx_bf16_to_f32(a.w_post[i]);
+        if (!a.w_next) return;
+        inv = statistics([&](int i) { return x[i]; }, 2, mean);
+        for (int i = tid; i < W; i += 256) {
+            const float v = (x[i] - mean) * inv * vmx_bf16_to_f32(a.w_next[i]);
+            if (a.h_f32) ((float *)a.h)[(int64_t)t * W + i] = v;
+            else ((uint16_t *)a.h)[(int64_t)t * W + i] = vmx_f32_to_bf16(v);
         }
-    } else {
-        for (int i = threadIdx.x; i < W; i += 256) store(i, x[i]);
     }
 }
 
@@ -409,11 +497,15 @@ int vmx_sandwich_norm(const VmxSandwich &a, int n, hipStream_t st) {
     VMX_REQUIRE(!a.w_next || a.h, "sandwich norm: the next norm needs its output rows");
     VMX_REQUIRE(!a.pair_rows || (a.pair_w && a.top >= 1), "sandwich norm: expert results need their weights");
     if (n <= 0) return VMX_OK;
-    if (a.width <= 256) hipLaunchKernelGGL(sandwich_norm_kernel<1>, dim3(n), dim3(256), 0, st, a);
-    else if (a.width <= 1024) hipLaunchKernelGGL(sandwich_norm_kernel<4>, dim3(n), dim3(256), 0, st, a);
-    else if (a.width <= 2048) hipLaunchKernelGGL(sandwich_norm_kernel<8>, dim3(n), dim3(256), 0, st, a);
-    else if (a.width <= 4096) hipLaunchKernelGGL(sandwich_norm_kernel<16>, dim3(n), dim3(256), 0, st, a);
-    else hipLaunchKernelGGL(sandwich_norm_kernel<0>, dim3(n), dim3(256), 0, st, a);
+    const bool vec = a.width % 4 == 0;   // every row then starts on a 16-byte (f32) / 8-byte (bf16) boundary
+#define SW(held, v) hipLaunchKernelGGL((sandwich_norm_kernel<held, v>), dim3(n), dim3(256), 0, st, a)
+    if (vec && a.width <= 1024) SW(1, 4);
+    else if (vec && a.width <= 2048) SW(2, 4);
+    else if (vec && a.width <= 4096) SW(4, 4);
+    else if (!vec && a.width <= 1024) SW(4, 1);
+    else if (!vec && a.width <= 4096) SW(16, 1);
+    else SW(0, 1);
+#undef SW
     VMX_CHECK_LAUNCH("sandwich norm");
     return VMX_OK;
 }
