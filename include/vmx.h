@@ -1331,6 +1331,8 @@ typedef struct vmx_matrix_memory_opts {
     int64_t ldgain;
     float *norm_out;              /* [tokens, ldnorm] per head: n . q with n <- g n + gain k carried beside S (NULL: none); the state then */
     int64_t ldnorm;               /* has vdim + 1 columns: vmx_gated_delta_rule_state_bytes(slots, heads, dim, vdim + 1) */
+    int bf16_operands;            /* the plain write with one decay per head may round q, k and v to bf16: steps of at least 8 tokens a */
+    int tokens;                   /* sequence (tokens: the step's rows) then run 64 tokens at a time on the matrix cores; all else stays f32 */
 } vmx_matrix_memory_opts;
 int vmx_matrix_memory_recurrence_ex(float *o, int64_t ldo, const float *q, int64_t ldq, float q_mul, const float *k, int64_t ldk,
                                     const float *v, int64_t ldv, const float *g, int64_t ldg, int g_per_head, const float *beta,

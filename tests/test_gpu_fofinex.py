@@ -319,9 +319,10 @@ def test_causal_latent_attention_with_a_needle(gpu, H, R, rd, dtype, bs):
         assert float((out.cpu().double() - want[a:b]).abs().max()) < tol, (a, b)
 
 
-def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul):
+def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul, chunks=False):
     """vmx_exp_gate_scan + vmx_matrix_memory_recurrence_ex over several sequences fed in unequal portions through slots that start
-    full of NaN.  Lists of [n, H, D], [n, H, D], [n, H, V], [n, H], [n, H]; per sequence [o / (max(|n . q|, e^-m) + 1e-6), o, n . q, e^-m]."""
+    full of NaN.  Lists of [n, H, D], [n, H, D], [n, H, V], [n, H], [n, H]; per sequence [o / (max(|n . q|, e^-m) + 1e-6), o, n . q, e^-m].
+    chunks: let steps with enough tokens take the chunked form (which rounds q, k and v to bf16)."""
     from vllm_rust_amd._lib import MatrixMemoryOpts, check, lib
     H, D, V = k[0].shape[1], k[0].shape[2], v[0].shape[2]
     nslots = max(slot_of) + 2
@@ -350,7 +351,7 @@ def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul):
         at = lambda off: x.data_ptr() + 4 * off   # noqa: E731
         check(lib.vmx_exp_gate_scan(at(oi), ld, at(oi + H), ld, floor.data_ptr(), H + 2, maxima.data_ptr(), cap, P.data_ptr(), S.data_ptr(), L.data_ptr(), len(slots),
                                     H, None))
-        mo = MatrixMemoryOpts(at(oi), ld, norm.data_ptr(), H + 1)
+        mo = MatrixMemoryOpts(at(oi), ld, norm.data_ptr(), H + 1, 1 if chunks else 0, T)
         check(lib.vmx_matrix_memory_recurrence_ex(o.data_ptr(), H * V, at(0), ld, q_mul, at(ok), ld, at(ov), ld, at(oi + H), ld, 1, None, 0, state.data_ptr(),
                                                   P.data_ptr(), S.data_ptr(), L.data_ptr(), len(slots), H, H, D, V, C.byref(mo), None))
         torch.cuda.synchronize()
@@ -366,17 +367,20 @@ def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul):
 
 @pytest.mark.parametrize("H,D,V,cap", [(2, 32, 32, 15.0), (3, 5, 7, 4.0), (4, 64, 47, 12.0), (1, 130, 16, 8.0), (2, 16, 1, 1.0), (5, 48, 64, 12.0)])
 @pytest.mark.parametrize("bias", [(0.0, 2.0), (-6.0, 0.0), (8.0, 4.0)])
-def test_exponential_memory_in_portions_through_dirty_slots(gpu, H, D, V, cap, bias):
-    """Three sequences of unequal length in portions of 1 .. 90 rows; input gates around zero, far below (the maximum then falls
+@pytest.mark.parametrize("chunks", [False, True])
+def test_exponential_memory_in_portions_through_dirty_slots(gpu, H, D, V, cap, bias, chunks):
+    """Both forms of the recurrence (with q, k and v that are bf16 numbers the chunked one is held to the same bounds; steps of few
+    tokens take the other form, so the two also hand the memory to each other).  Three sequences of unequal length in portions of 1 .. 90 rows; input gates around zero, far below (the maximum then falls
     from its start at 0 and the floor e^-m counts) and far above."""
     _, torch = gpu
     from tests import fofinex_oracle as orc
     gen = torch.Generator().manual_seed(H * D + V)
-    lens = [131, 1, 70]
+    lens = [331, 1, 70]
     rn = lambda *s: torch.randn(*s, generator=gen, dtype=torch.float64).float().double()   # noqa: E731
-    q, k, v = [rn(n, H, D) for n in lens], [rn(n, H, D) for n in lens], [rn(n, H, V) for n in lens]
+    bf = lambda *s: rn(*s).to(torch.bfloat16).double()   # noqa: E731
+    q, k, v = [bf(n, H, D) for n in lens], [bf(n, H, D) for n in lens], [bf(n, H, V) for n in lens]
     zi, zf = [(2 * rn(n, H) + bias[0]).float().double() for n in lens], [(2 * rn(n, H) + bias[1]).float().double() for n in lens]
-    got = _run_exp_memory(torch, q, k, v, zi, zf, cap, [[90, 1, 1, 37, 2], [1], [2, 3, 63, 1, 1]], [3, 0, 4], D ** -0.5)
+    got = _run_exp_memory(torch, q, k, v, zi, zf, cap, [[90, 1, 1, 37, 2, 200], [1], [2, 3, 63, 1, 1]], [3, 0, 4], D ** -0.5, chunks)
     for s in range(3):
         parts = []
         want = orc.exponential_gate_memory(q[s] * D ** -0.5, k[s], v[s], *orc.log_gates(zi[s], zf[s], cap), parts)
@@ -389,7 +393,8 @@ def test_exponential_memory_in_portions_through_dirty_slots(gpu, H, D, V, cap, b
         assert float(((got[s][0] - want) * sound).abs().max()) < 1e-3 * max(1.0, float((want * sound).abs().max())), s
 
 
-def test_exponential_memory_keeps_a_far_key_and_starts_at_zero(gpu):
+@pytest.mark.parametrize("chunks", [False, True])
+def test_exponential_memory_keeps_a_far_key_and_starts_at_zero(gpu, chunks):
     """A key written at position 5 with the largest input gate and asked for 290 tokens and four portions later, through a forget
     gate of nearly one on head 0 and of one half on head 1; before it the memory is empty of it.  The first token's floor is
     e^-max(f, i), which leaves a small write small."""
@@ -398,21 +403,21 @@ def test_exponential_memory_keeps_a_far_key_and_starts_at_zero(gpu):
     n, D, V, cap = 300, 16, 8, 10.0
     gen = torch.Generator().manual_seed(0)
     k = torch.zeros(n, 2, D, dtype=torch.float64)
-    k[:, :, 1:] = torch.randn(n, 2, D - 1, generator=gen, dtype=torch.float64).float().double()
+    k[:, :, 1:] = torch.randn(n, 2, D - 1, generator=gen, dtype=torch.float64).to(torch.bfloat16).double()
     k[5, :, 0] = 1.0
-    v = torch.randn(n, 2, V, generator=gen, dtype=torch.float64).float().double()
+    v = torch.randn(n, 2, V, generator=gen, dtype=torch.float64).to(torch.bfloat16).double()
     q = torch.zeros(n, 2, D, dtype=torch.float64)
     q[:, :, 0] = 1.0
     zi, zf = torch.full((n, 2), -4.0, dtype=torch.float64), torch.zeros(n, 2, dtype=torch.float64)
     zi[5], zf[:, 0] = 6.0, 90.0
-    got = _run_exp_memory(torch, [q], [k], [v], [zi], [zf], cap, [[4, 100, 1, 150, 45]], [1], 1.0)[0][0]
+    got = _run_exp_memory(torch, [q], [k], [v], [zi], [zf], cap, [[4, 100, 1, 150, 45]], [1], 1.0, chunks)[0][0]
     want = orc.exponential_gate_memory(q, k, v, *orc.log_gates(zi, zf, cap))
     assert float(got[:5].abs().max()) == 0 and float((got - want).abs().max()) < 1e-5
     for t in (5, 6, 104, 105, 295, 299):
         assert float((got[t, 0] - v[5, 0]).abs().max()) < 0.05 * float(v[5, 0].abs().max())      # still there, nearly whole
     assert float(got[40:, 1].abs().max()) < 1e-3 * float(v[5, 1].abs().max())
     k[0, :, 0] = 1.0                                                                               # the very first token, a small input gate
-    got = _run_exp_memory(torch, [q[:1]], [k[:1]], [v[:1]], [zi[:1]], [zf[:1]], cap, [[1]], [0], 1.0)[0][0]
+    got = _run_exp_memory(torch, [q[:1]], [k[:1]], [v[:1]], [zi[:1]], [zf[:1]], cap, [[1]], [0], 1.0, chunks)[0][0]
     m = torch.maximum(orc.log_gates(zi[0], zf[0], cap)[1], orc.log_gates(zi[0], zf[0], cap)[0])
     w = torch.exp(orc.log_gates(zi[0], zf[0], cap)[0])
     assert float((got[0] - v[0] * (w / torch.maximum(w, torch.ones(2, dtype=torch.float64))).unsqueeze(-1)).abs().max()) < 1e-5 and float(m[1]) < 0

@@ -394,7 +394,7 @@ class LatentPrepare(C.Structure):
 
 class MatrixMemoryOpts(C.Structure):
     """struct vmx_matrix_memory_opts (include/vmx.h)."""
-    _fields_ = [("write_gain", _p), ("ldgain", _i64), ("norm_out", _p), ("ldnorm", _i64)]
+    _fields_ = [("write_gain", _p), ("ldgain", _i64), ("norm_out", _p), ("ldnorm", _i64), ("bf16_operands", _i), ("tokens", _i)]
 
 
 class ReadOutOpts(C.Structure):

@@ -18,7 +18,8 @@
 // head of value head h: h / (heads / qk_heads).  A workgroup owns 16 value columns of one (sequence, head) and walks the
 // sequence's tokens of the step in order; 16 threads share a column, each holding every 16th row of S in registers, and the
 // column sums per token are 16-lane butterflies.  The state slot keeps S in the workgroup's own register order (the layout is
-// private to this kernel), so that loading and storing it is coalesced.
+// private to this file), so that loading and storing it is coalesced.  Prompts of the plain memory with one decay per head have a
+// chunked form on the matrix cores below, over the same state layout.
 //
 // Exponential gates (vmx_exp_gate_scan): a memory whose input gate is an exponential keeps the logarithm of its scale, a running
 // maximum m_t = max(f_t + m_(t-1), i_t) per head (from 0), in its slot; what the recurrence needs are the decay
@@ -269,6 +270,250 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(const DeltaArgs a
     for (int u = 0; u < DPT; u++) sp[(int64_t)u * 256] = S[u];
 }
 
+// ---------------------------------------------------------------------------------------------------------------------------
+// Chunked matrix-core form of the plain memory with one decay per head (S <- g_t S + a_t k_t v_t^T), for prompts.  A workgroup owns
+// the same 16 value columns of one (sequence, head) as above and walks the sequence's tokens of the step 64 at a time; with
+// L_t = sum of log g up to token t of the chunk and S the memory ahead of it,
+//   o_t = e^(L_t) S^T q_t + sum_(s <= t) a_s e^(L_t - L_s) (q_t . k_s) v_s
+//   S  <- e^(L_C) S + sum_s k_s (a_s e^(L_C - L_s) v_s)^T
+// are four small products per chunk (v_mfma_f32_16x16x32_bf16).  q, k and v are rounded to bf16; everything else is f32: a number
+// that is not a bf16 enters a product as the sum of three bf16 parts (24 bits), so the memory, the weighted scores and the weighted
+// values keep f32 precision.  L is summed in double (a chunk may cross decays of e^-80, whose differences still count).
+// Wave w takes tokens 16 w .. 16 w + 15 of the first two products and rows w, w + 4, ... of 16 of the memory in the last.
+constexpr int MC_C = 64, MC_LD = MC_C + 8;
+
+struct MemoryChunkLds {   // offsets in bytes
+    int q, k, p, v, wv, s, gates, total, dp, ldq, ldk;
+};
+__host__ __device__ constexpr MemoryChunkLds memory_chunk_lds(int dt) {
+    MemoryChunkLds l{};
+    l.dp = 16 * dt, l.ldq = l.dp + 8, l.ldk = l.dp + 32;
+    l.q = 0;
+    l.k = l.q + MC_C * l.ldq * 2;
+    l.p = l.k + MC_C * l.ldk * 2;
+    l.v = l.p + 3 * MC_C * MC_LD * 2;
+    l.wv = l.v + 16 * MC_LD * 2;
+    l.s = l.wv + 3 * 16 * MC_LD * 2;
+    l.gates = l.s + 3 * 16 * l.ldq * 2;
+    l.total = l.gates + 2 * MC_C * (8 + 3 * 4) + 2 * 4;
+    return l;
+}
+typedef short mc_s16x4 __attribute__((ext_vector_type(4)));
+typedef short mc_s16x8 __attribute__((ext_vector_type(8)));
+
+__device__ __forceinline__ void mc_split(float x, uint16_t (&p)[3]) {   // x = p0 + p1 + p2 to 24 bits
+#pragma unroll
+    for (int i = 0; i < 3; i++) {
+        p[i] = vmx_f32_to_bf16(x);
+        x -= vmx_bf16_to_f32(p[i]);
+    }
+}
+__device__ __forceinline__ vmx_f32x4 mc_mfma(const uint4 a, const uint4 b, vmx_f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(vmx_bf16x8, a), __builtin_bit_cast(vmx_bf16x8, b), c, 0, 0, 0);
+}
+
+template <int DT> __global__ __launch_bounds__(256) void memory_chunk_kernel(const DeltaArgs a) {
+    constexpr MemoryChunkLds l = memory_chunk_lds(DT);
+    constexpr int DP = l.dp, NQ = MC_C * DP / 4 / 256, ST = DT / 4, KS = DP / 32;
+    extern __shared__ __align__(16) unsigned char mc_lds[];
+    uint16_t *Q = (uint16_t *)(mc_lds + l.q), *K = (uint16_t *)(mc_lds + l.k), *P = (uint16_t *)(mc_lds + l.p), *V = (uint16_t *)(mc_lds + l.v),
+             *WV = (uint16_t *)(mc_lds + l.wv), *SS = (uint16_t *)(mc_lds + l.s);
+    double *gl = (double *)(mc_lds + l.gates);                    // [2][C] L
+    float *ga = (float *)(gl + 2 * MC_C), *gw = ga + 2 * MC_C, *gc = gw + 2 * MC_C, *gt = gc + 2 * MC_C;   // [2][C] a, a e^(L_C - L), e^L; [2] e^(L_C)
+    const int seq = blockIdx.z, h = blockIdx.y, tile = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fl = lane & 15, fg = lane >> 4;
+    const int first = a.seq_starts[seq], count = a.seq_starts[seq + 1] - first;
+    if (count <= 0) return;
+    const int qh = h / (a.heads / a.qk_heads);
+    const float *qp = a.q + (int64_t)first * a.ldq + (int64_t)qh * a.dim, *kp = a.k + (int64_t)first * a.ldk + (int64_t)qh * a.dim;
+    const float *vp = a.v + (int64_t)first * a.ldv + (int64_t)h * a.vdim;
+    const bool vec = (a.dim & 3) == 0 && (a.ldq & 3) == 0 && (a.ldk & 3) == 0 && (((uintptr_t)qp | (uintptr_t)kp) & 15) == 0;
+    // ---- what a thread stages: NQ groups of four q / k channels, four value columns of one token, and (wave 0) a token's gates
+    float4 rq[NQ], rk[NQ];
+    float rv[4], g1 = 1.f, a1 = 0.f;
+    const int vt = tid >> 2, vc = 4 * (tid & 3);
+    auto four = [&](const float *p, int64_t ld, int t, int d) {
+        if (t >= count || d >= a.dim) return make_float4(0.f, 0.f, 0.f, 0.f);
+        p += (int64_t)t * ld + d;
+        if (vec) return *reinterpret_cast<const float4 *>(p);
+        return make_float4(p[0], d + 1 < a.dim ? p[1] : 0.f, d + 2 < a.dim ? p[2] : 0.f, d + 3 < a.dim ? p[3] : 0.f);
+    };
+    auto request = [&](int t0) {
+#pragma unroll
+        for (int j = 0; j < NQ; j++) {
+            const int i = tid + 256 * j, t = t0 + i / (DP / 4), d = 4 * (i % (DP / 4));
+            rq[j] = four(qp, a.ldq, t, d);
+            rk[j] = four(kp, a.ldk, t, d);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int c = tile * DR_VT + vc + e;
+            rv[e] = t0 + vt >= count ? 0.f : (c < a.vdim ? vp[(int64_t)(t0 + vt) * a.ldv + c] : (c == a.vdim && a.norm ? 1.f : 0.f));
+        }
+    };
+    auto request_gates = [&](int t0) {   // wave 0
+        const int t = t0 + lane;
+        g1 = t < count ? a.g[(int64_t)(first + t) * a.ldg + h] : 1.f;
+        a1 = t < count ? (a.beta ? a.beta[(int64_t)(first + t) * a.ldbeta + h] : 1.f) : 0.f;
+    };
+    auto scan_gates = [&](int b) {       // wave 0: L and what follows from it for the chunk whose gates it holds
+        double L = log((double)fmaxf(g1, 1e-37f));
+#pragma unroll
+        for (int d = 1; d < 64; d <<= 1) {
+            const double p = __shfl_up(L, d, 64);
+            if (lane >= d) L += p;
+        }
+        const double end = __shfl(L, 63, 64);
+        gl[b * MC_C + lane] = L;
+        ga[b * MC_C + lane] = a1;
+        gw[b * MC_C + lane] = a1 * expf((float)(end - L));
+        gc[b * MC_C + lane] = expf((float)L) * a.q_mul;
+        if (lane == 0) gt[b] = expf((float)end);
+    };
+    auto store4 = [](uint16_t *dst, const float4 f) {
+        *reinterpret_cast<uint2 *>(dst) = make_uint2((uint32_t)vmx_f32_to_bf16(f.x) | ((uint32_t)vmx_f32_to_bf16(f.y) << 16),
+                                                     (uint32_t)vmx_f32_to_bf16(f.z) | ((uint32_t)vmx_f32_to_bf16(f.w) << 16));
+    };
+    float vv[4];
+    auto stage = [&]() {
+#pragma unroll
+        for (int j = 0; j < NQ; j++) {
+            const int i = tid + 256 * j, t = i / (DP / 4), d = 4 * (i % (DP / 4));
+            store4(Q + t * l.ldq + d, rq[j]);
+            store4(K + t * l.ldk + d, rk[j]);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const uint16_t r = vmx_f32_to_bf16(rv[e]);
+            V[(vc + e) * MC_LD + vt] = r;
+            vv[e] = vmx_bf16_to_f32(r);
+        }
+    };
+    // ---- the memory: rows 16 u + 4 fg + r (u = wave + 4 j), column fl, in registers; its three parts by column in LDS
+    float *sp = a.state + ((((int64_t)a.state_slots[seq] * a.heads + h) * gridDim.x + tile) * DT) * 256 + fl * 16 + 4 * fg;
+    const bool fresh = a.positions[first] == 0;
+    vmx_f32x4 S[ST];
+    auto split_memory = [&]() {
+#pragma unroll
+        for (int j = 0; j < ST; j++) {
+            uint16_t p[4][3];
+#pragma unroll
+            for (int r = 0; r < 4; r++) mc_split(S[j][r], p[r]);
+#pragma unroll
+            for (int i = 0; i < 3; i++)
+                *reinterpret_cast<uint2 *>(SS + (i * 16 + fl) * l.ldq + 16 * (wave + 4 * j) + 4 * fg) =
+                    make_uint2((uint32_t)p[0][i] | ((uint32_t)p[1][i] << 16), (uint32_t)p[2][i] | ((uint32_t)p[3][i] << 16));
+        }
+    };
+    request(0);
+    if (wave == 0) request_gates(0);
+#pragma unroll
+    for (int j = 0; j < ST; j++) {
+        const float4 f = fresh ? make_float4(0.f, 0.f, 0.f, 0.f) : *reinterpret_cast<const float4 *>(sp + (wave + 4 * j) * 256);
+        S[j] = vmx_f32x4{f.x, f.y, f.z, f.w};
+    }
+    split_memory();
+    for (int i = tid; i < 3 * MC_C * MC_LD / 4; i += 256) reinterpret_cast<uint2 *>(P)[i] = make_uint2(0, 0);   // scores after the diagonal block stay 0
+    stage();
+    if (wave == 0) {
+        scan_gates(0);
+        request_gates(MC_C);
+    }
+    for (int t0 = 0, b = 0; t0 < count; t0 += MC_C, b ^= 1) {
+        __syncthreads();
+        const bool more = t0 + MC_C < count;
+        if (more) request(t0 + MC_C);
+        if (wave == 0 && more) {
+            scan_gates(b ^ 1);
+            request_gates(t0 + 2 * MC_C);
+        }
+        // values times their weight at the chunk's end, in three parts
+        {
+            const float w = gw[b * MC_C + vt];
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                uint16_t p[3];
+                mc_split(w * vv[e], p);
+#pragma unroll
+                for (int i = 0; i < 3; i++) WV[(i * 16 + vc + e) * MC_LD + vt] = p[i];
+            }
+        }
+        // scores of this wave's tokens against the chunk's keys up to them, weighted, in three parts
+        uint4 qf[KS];
+#pragma unroll
+        for (int ks = 0; ks < KS; ks++) qf[ks] = *reinterpret_cast<const uint4 *>(Q + (16 * wave + fl) * l.ldq + 32 * ks + 8 * fg);
+        double Lt[4];
+#pragma unroll
+        for (int r = 0; r < 4; r++) Lt[r] = gl[b * MC_C + 16 * wave + 4 * fg + r];
+        for (int j = 0; j <= wave; j++) {
+            vmx_f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) sc = mc_mfma(qf[ks], *reinterpret_cast<const uint4 *>(K + (16 * j + fl) * l.ldk + 32 * ks + 8 * fg), sc);
+            const int sidx = 16 * j + fl;
+            const double Ls = gl[b * MC_C + sidx];
+            const float as = ga[b * MC_C + sidx] * a.q_mul;
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int t = 16 * wave + 4 * fg + r;
+                uint16_t p[3];
+                mc_split(sidx <= t ? sc[r] * as * expf((float)(Lt[r] - Ls)) : 0.f, p);
+#pragma unroll
+                for (int i = 0; i < 3; i++) P[(i * MC_C + t) * MC_LD + sidx] = p[i];
+            }
+        }
+        // o = e^L q . S (the memory ahead of the chunk) + weighted scores . v
+        vmx_f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 2; i >= 0; i--)
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) o = mc_mfma(qf[ks], *reinterpret_cast<const uint4 *>(SS + (i * 16 + fl) * l.ldq + 32 * ks + 8 * fg), o);
+#pragma unroll
+        for (int r = 0; r < 4; r++) o[r] *= gc[b * MC_C + 16 * wave + 4 * fg + r];
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");   // the wave's own rows of P
+        for (int ks = 0; ks < (wave >> 1) + 1; ks++) {
+            const uint4 vf = *reinterpret_cast<const uint4 *>(V + fl * MC_LD + 32 * ks + 8 * fg);
+#pragma unroll
+            for (int i = 2; i >= 0; i--) o = mc_mfma(*reinterpret_cast<const uint4 *>(P + (i * MC_C + 16 * wave + fl) * MC_LD + 32 * ks + 8 * fg), vf, o);
+        }
+        const int c = tile * DR_VT + fl;
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const int t = t0 + 16 * wave + 4 * fg + r;
+            if (t < count) {
+                if (c < a.vdim) a.o[(int64_t)(first + t) * a.ldo + (int64_t)h * a.vdim + c] = o[r];
+                else if (c == a.vdim && a.norm) a.norm[(int64_t)(first + t) * a.ldnorm + h] = o[r];
+            }
+        }
+        __syncthreads();
+        // the memory after the chunk
+        const float gall = gt[b];
+#pragma unroll
+        for (int j = 0; j < ST; j++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) S[j][r] *= gall;
+#pragma unroll
+        for (int ks = 0; ks < MC_C / 32; ks++) {
+            uint4 wf[3];
+#pragma unroll
+            for (int i = 0; i < 3; i++) wf[i] = *reinterpret_cast<const uint4 *>(WV + (i * 16 + fl) * MC_LD + 32 * ks + 8 * fg);
+#pragma unroll
+            for (int j = 0; j < ST; j++) {
+                // A operand = K^T: the transposing LDS read hands lane n channel 16 u + n of the four tokens its 16-lane group addressed
+                const uint16_t *src = K + (32 * ks + 8 * fg + (fl >> 2)) * l.ldk + 16 * (wave + 4 * j) + 4 * (fl & 3);
+                const mc_s16x4 c0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((mc_s16x4 __attribute__((address_space(3))) *)src);
+                const mc_s16x4 c1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((mc_s16x4 __attribute__((address_space(3))) *)(src + 4 * l.ldk));
+                const uint4 kf = __builtin_bit_cast(uint4, mc_s16x8{c0[0], c0[1], c0[2], c0[3], c1[0], c1[1], c1[2], c1[3]});
+#pragma unroll
+                for (int i = 2; i >= 0; i--) S[j] = mc_mfma(kf, wf[i], S[j]);
+            }
+        }
+        if (more) split_memory();
+        __syncthreads();
+        if (more) stage();
+    }
+#pragma unroll
+    for (int j = 0; j < ST; j++) *reinterpret_cast<float4 *>(sp + (wave + 4 * j) * 256) = make_float4(S[j][0], S[j][1], S[j][2], S[j][3]);
+}
+
 // In place, one workgroup per (sequence, head): i[t, h] <- exp(i_t - m_t), f[t, h] <- exp(f_t + m_(t-1) - m_t), floor[t, h] = exp(-m_t)
 // with i_t = cap tanh(i / cap), f_t = log(sigmoid(cap tanh(f / cap))) and m the running maximum (the slot's; 0 at position 0).
 __global__ __launch_bounds__(256) void exp_gate_scan_kernel(float *__restrict__ ig, int64_t ldi, float *__restrict__ fg, int64_t ldf,
@@ -407,6 +652,16 @@ static size_t delta_lds_bytes(int dpt) {
     const size_t ct = 128 / dpt, row = (size_t)DR_RS * (dpt == 4 ? 4 : dpt + 4);
     return (3 * 2 * ct * row + 2 * ct * DR_VT + 2 * ct) * 4;
 }
+template <int DT> static int memory_chunk_launch(const DeltaArgs &a, dim3 grid, hipStream_t st) {
+    static bool sized = false;
+    constexpr int lds = memory_chunk_lds(DT).total;
+    if (!sized) {
+        VMX_CHECK_HIP(hipFuncSetAttribute((const void *)memory_chunk_kernel<DT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+        sized = true;
+    }
+    hipLaunchKernelGGL(memory_chunk_kernel<DT>, grid, dim3(256), lds, st, a);
+    return VMX_OK;
+}
 template <int DPT> static int delta_launch(const DeltaArgs &a, dim3 grid, hipStream_t st) {
     static bool sized = false;   // more than 64 KiB of LDS has to be asked for once per kernel
     const size_t lds = delta_lds_bytes(DPT);
@@ -468,6 +723,17 @@ extern "C" int vmx_matrix_memory_recurrence_ex(float *o, int64_t ldo, const floa
     const dim3 grid((vdim + (norm ? 1 : 0) + DR_VT - 1) / DR_VT, heads, num_seqs);
     hipStream_t st = vmx_stream(stream);
     int rc;
+    // prompts: 64 tokens at a time on the matrix cores, where the caller takes q, k and v in bf16
+    if (opts && opts->bf16_operands && !beta && g_per_head && opts->tokens >= 8 * num_seqs) {
+        switch (delta_dpt(dim)) {
+            case 4: rc = memory_chunk_launch<4>(a, grid, st); break;
+            case 8: rc = memory_chunk_launch<8>(a, grid, st); break;
+            default: rc = memory_chunk_launch<16>(a, grid, st); break;
+        }
+        if (rc) return rc;
+        VMX_CHECK_LAUNCH("matrix_memory_recurrence (chunks)");
+        return VMX_OK;
+    }
     switch (delta_dpt(dim)) {
         case 4: rc = delta_launch<4>(a, grid, st); break;
         case 8: rc = delta_launch<8>(a, grid, st); break;

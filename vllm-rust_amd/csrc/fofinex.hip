@@ -395,7 +395,7 @@ int exp_memory(vmx_fofinex *m, Layer &L, const Step &s) {
     if (int rc = vmx_exp_gate_scan(gain, nf, decay, nf, m->floor.as<float>(), H, L.maxima.as<float>(), lc.gate_cap, s.positions, s.seq_starts,
                                    s.state_slots, s.num_seqs, H, s.st))
         return rc;
-    const vmx_matrix_memory_opts mo = {gain, nf, m->norm.as<float>(), H};
+    const vmx_matrix_memory_opts mo = {gain, nf, m->norm.as<float>(), H, f32 ? 0 : 1, T};
     if (int rc = vmx_matrix_memory_recurrence_ex(m->readout.as<float>(), (int64_t)H * V, fused + L.q_off, nf, 1.0f / sqrtf((float)D), fused + L.k_off, nf,
                                                  fused + L.v_off, nf, decay, nf, 1, nullptr, 0, L.memory.as<float>(), s.positions, s.seq_starts,
                                                  s.state_slots, s.num_seqs, H, H, D, V, &mo, s.st))
