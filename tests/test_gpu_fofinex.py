@@ -164,7 +164,7 @@ def feed(engine, seq_id, toks, cuts, finish=True):
 
 # ----------------------------------------------------------------------------- mechanisms alone
 
-@pytest.mark.parametrize("E,top,groups,keep", [(16, 3, 4, 3), (12, 2, 3, 1), (8, 8, 4, 4), (70, 4, 7, 2), (256, 6, 16, 4), (6, 2, 6, 3), (5, 2, 1, 1), (64, 1, 2, 1),
+@pytest.mark.parametrize("E,top,groups,keep", [(20, 3, 5, 3), (12, 2, 3, 1), (8, 8, 4, 4), (70, 4, 7, 2), (256, 6, 16, 4), (6, 2, 6, 3), (5, 2, 1, 1), (64, 1, 2, 1),
                                                (1, 1, 1, 1), (200, 12, 2, 2)])
 @pytest.mark.parametrize("shift", [0.0, -0.9, 0.4])
 def test_corrected_router(gpu, E, top, groups, keep, shift):
@@ -211,7 +211,7 @@ def test_corrected_router_ties_and_group_sums(gpu):
     assert run([-1.0, -2.0, -1.5, -1.25, -4.0, -0.5], 3, 3, 2) == [0, 3, 2]
 
 
-@pytest.mark.parametrize("H,dim,rd,rdims,R,Q,stretch", [(3, 10, 6, 6, 20, 18, True), (6, 64, 32, 32, 128, 80, True), (2, 0, 8, 8, 16, 5, False), (4, 7, 10, 4, 33, 7, False),
+@pytest.mark.parametrize("H,dim,rd,rdims,R,Q,stretch", [(3, 10, 6, 6, 20, 18, True), (5, 64, 24, 24, 112, 72, True), (2, 0, 8, 8, 16, 5, False), (4, 7, 10, 4, 33, 7, False),
                                                         (1, 16, 0, 0, 24, 300, False), (2, 4, 300, 300, 512, 1, True)])
 @pytest.mark.parametrize("dtype", [0, 1])
 def test_latent_preparation_part_by_part(gpu, H, dim, rd, rdims, R, Q, stretch, dtype):
@@ -274,7 +274,7 @@ def test_latent_preparation_part_by_part(gpu, H, dim, rd, rdims, R, Q, stretch, 
     assert float((qlo[:-1].reshape(T, Q) - orc.rms_unit(ql[:, :Q].double(), eps) * qn.double()).abs().max()) < 1e-5 + low
 
 
-@pytest.mark.parametrize("H,R,rd", [(3, 24, 8), (6, 128, 32), (16, 64, 16), (20, 16, 0), (2, 33, 6), (5, 256, 64)])
+@pytest.mark.parametrize("H,R,rd", [(3, 24, 8), (7, 112, 40), (16, 64, 16), (20, 16, 0), (2, 33, 6), (5, 256, 64)])
 @pytest.mark.parametrize("dtype,bs", [(0, 16), (1, 16), (1, 5), (0, 1)])
 def test_causal_latent_attention_with_a_needle(gpu, H, R, rd, dtype, bs):
     """No window: one key whose score stands out is found from its own position to 400 keys later, at page borders, as the first
@@ -365,7 +365,7 @@ def _run_exp_memory(torch, q, k, v, zi, zf, cap, portions, slot_of, q_mul, chunk
     return [[torch.cat([x[j] for x in g]) for j in range(4)] for g in got]
 
 
-@pytest.mark.parametrize("H,D,V,cap", [(2, 32, 32, 15.0), (3, 5, 7, 4.0), (4, 64, 47, 12.0), (1, 130, 16, 8.0), (2, 16, 1, 1.0), (5, 48, 64, 12.0)])
+@pytest.mark.parametrize("H,D,V,cap", [(2, 32, 32, 15.0), (3, 5, 7, 4.0), (4, 64, 47, 11.0), (1, 130, 16, 8.0), (2, 16, 1, 1.0), (6, 40, 56, 10.0)])
 @pytest.mark.parametrize("bias", [(0.0, 2.0), (-6.0, 0.0), (8.0, 4.0)])
 @pytest.mark.parametrize("chunks", [False, True])
 def test_exponential_memory_in_portions_through_dirty_slots(gpu, H, D, V, cap, bias, chunks):
@@ -681,7 +681,7 @@ def random_spec(rng):
         else:
             ff = dict(mlp="dense", ff=size(5, 70)) if kind == "dense" else dict(mlp=None)
         if rng.random() < 0.5:
-            layers.append(mem_layer(heads=int(rng.integers(1, 6)), dim=size(3, 60), vdim=size(4, 50), gate_cap=float(pick(3.0, 12.0, 15.0)), **ff))   # a norm over 1 .. 3 numbers turns rounding into sign flips
+            layers.append(mem_layer(heads=int(rng.integers(1, 6)), dim=size(3, 60), vdim=size(4, 50), gate_cap=float(pick(3.0, 10.0, 15.0)), **ff))   # a norm over 1 .. 3 numbers turns rounding into sign flips
             continue
         own = [j for j, l in enumerate(layers) if l.mixer == "latent_attention" and l.kv_from is None]
         a = dict(heads=int(rng.integers(1, 8)), dim=size(2, 40), vdim=size(3, 40), q_rank=size(5, 40), scale=float(rng.uniform(0.1, 0.5)), **ff)
