@@ -1134,6 +1134,7 @@ typedef struct vmx_window_attn_extras {
     const uint16_t *dist_r2_bf16;
     const uint16_t *talk_bf16;      /* [heads, heads]: score_h <- sum_g talk[h, g] score_g over the visible keys, before the softmax */
     int gate_per_element;           /* the gate rows hold heads * vdim numbers (one per output element) instead of one per head */
+    int chunk;                      /* > 0: position i sees only keys j with floor(j / chunk) = floor(i / chunk) (and the kept first tokens) */
 } vmx_window_attn_extras;
 /* vmx_window_attention with these extras (NULL: none).  Order: scale and temperature, soft cap, distance penalty, mixing of the
  * heads, mask, softmax (with sink), weighted sum, gate.  Mixing needs heads <= 64 and heads * dim <= 8192. */
@@ -1206,7 +1207,8 @@ int vmx_topk_sigmoid(const float *logits, float *topk_weights, int32_t *topk_ids
 
 /* What vmx_qk_prepare_ex does differently from vmx_qk_prepare_cache_write. */
 typedef struct vmx_qk_prepare_opts {
-    int norm_per_head;    /* the norms run over each head of head_dim numbers; the gains hold head_dim numbers, the same for every head */
+    int norm_per_head;    /* the norms run over each head of head_dim numbers, with head_dim gains, the same for every head (0: over the whole
+                             row, with a gain per number) */
     int rot_halves;       /* coordinate i turns with i + rot_dims / 2 (i < rot_dims / 2) instead of 2i with 2i + 1 */
     float rot_mul;        /* cos and sin are multiplied by this (0: 1) */
     float q_mul, k_mul;   /* constant multipliers of the prepared queries / keys, after the rotation (0: 1) */
@@ -1407,6 +1409,51 @@ int vmx_fofinex_forward(vmx_fofinex *m, const int32_t *tokens, const int32_t *po
                         int num_tokens, const int32_t *block_tables, int num_seqs, int max_blocks_per_seq, const int32_t *seq_starts,
                         const int32_t *state_slots, const int32_t *logit_rows, int num_logit_rows, float *logits, int32_t *greedy_ids,
                         float *layer_trace, void *stream);
+
+/* ------------------------------------------------------- chunked attention beside a decayed matrix memory, Larolorn executor */
+
+#define VMX_MIXER_CHUNKED_LIGHTNING 9    /* chunked sink attention (whole-row q / k norms) beside a memory with one constant decay per head */
+#define VMX_MLP_CLAMPED_GLU 8            /* g sigmoid(1.702 g) (u + 1), gate and up values clamped */
+
+/* One layer of a Larolorn model: x <- x + m N1(mixer(x)); x <- x + m N2(ff(x)), N an RMS norm with a gain (ff may be absent). */
+typedef struct vmx_larolorn_layer_config {
+    int mixer;                    /* VMX_MIXER_LATENT_ATTENTION or VMX_MIXER_CHUNKED_LIGHTNING */
+    int heads, dim, vdim;         /* latent attention: dim unrotated query/key coordinates; otherwise the left attention's */
+    float scale;                  /* score scale */
+    int mask;                     /* latent attention: window; left attention: chunk (0: every earlier key) */
+    vmx_rotation rot;             /* latent attention: neighbours of the rot_dim part; left attention: halves (dims 0: none) */
+    int rot_dim, kv_rank;         /* latent attention */
+    int kv_heads;                 /* left attention */
+    int r_heads, r_dim, r_vdim;   /* right side: heads, key and value sizes */
+    const float *decay;           /* right side: host array of r_heads decays (read during create) */
+    int mlp;                      /* VMX_MLP_NONE or VMX_MLP_CLAMPED_GLU */
+    int ff;
+    float limit;
+    int weights_of;               /* the layer whose weights it runs with, cache and state being its own (-1: its own weights) */
+} vmx_larolorn_layer_config;
+
+typedef struct vmx_larolorn_config {
+    int vocab, width, num_layers;
+    float norm_eps, residual_mult, logit_scale;
+    int dtype;                    /* VMX_BF16: bf16 operands and cache; VMX_F32: everything in f32 */
+    int block_size, num_blocks;   /* paged caches: rows per block, blocks per layer */
+    int max_tokens, max_seqs;     /* most tokens / sequences of one forward call */
+    int state_slots;              /* recurrent-state slots (one per live sequence) */
+} vmx_larolorn_config;
+
+typedef struct vmx_larolorn vmx_larolorn;
+int vmx_larolorn_create(const vmx_larolorn_config *cfg, const vmx_larolorn_layer_config *layers, vmx_larolorn **out);
+void vmx_larolorn_destroy(vmx_larolorn *m);
+/* One checkpoint tensor under its name in the file: "embed", "head", "final.norm", "l<i>.norm1|norm2"; latent attention
+ * "l<i>.mix.q|dkv|dkv.norm|uk|uv|g|o"; two-sided "l<i>.mix.left.q|k|v|o" (+ ".b"), "mix.left.q.norm|k.norm|sink|out",
+ * "l<i>.mix.right.q|k|v|g|o|norm|out"; "l<i>.mlp.gate|up|down": bf16, matrices [out, in]; host or device memory. */
+int vmx_larolorn_load_tensor(vmx_larolorn *m, const char *name, const void *data, size_t bytes, void *stream);
+int vmx_larolorn_missing_tensors(const vmx_larolorn *m);
+/* One step over packed tokens, arguments as vmx_gupuvik_forward. */
+int vmx_larolorn_forward(vmx_larolorn *m, const int32_t *tokens, const int32_t *positions, const int32_t *slots, const int32_t *seq_ids,
+                         int num_tokens, const int32_t *block_tables, int num_seqs, int max_blocks_per_seq, const int32_t *seq_starts,
+                         const int32_t *state_slots, const int32_t *logit_rows, int num_logit_rows, float *logits, int32_t *greedy_ids,
+                         float *layer_trace, void *stream);
 
 #ifdef __cplusplus
 }

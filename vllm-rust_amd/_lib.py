@@ -267,6 +267,11 @@ _SIGS = {
     "vmx_fofinex_load_tensor": (_i, [_p, C.c_char_p, _p, _sz, _p]),
     "vmx_fofinex_missing_tensors": (_i, [_p]),
     "vmx_fofinex_forward": (_i, [_p, _p, _p, _p, _p, _i, _p, _i, _i, _p, _p, _p, _i, _p, _p, _p, _p]),
+    "vmx_larolorn_create": (_i, [_p, _p, _p]),
+    "vmx_larolorn_destroy": (None, [_p]),
+    "vmx_larolorn_load_tensor": (_i, [_p, C.c_char_p, _p, _sz, _p]),
+    "vmx_larolorn_missing_tensors": (_i, [_p]),
+    "vmx_larolorn_forward": (_i, [_p, _p, _p, _p, _p, _i, _p, _i, _i, _p, _p, _p, _i, _p, _p, _p, _p]),
 }
 
 
@@ -335,7 +340,7 @@ class GupuvikConfig(C.Structure):
 
 class WindowAttnExtras(C.Structure):
     """struct vmx_window_attn_extras (include/vmx.h)."""
-    _fields_ = [("sink_bf16", _p), ("dist_r1_bf16", _p), ("dist_r2_bf16", _p), ("talk_bf16", _p), ("gate_per_element", _i)]
+    _fields_ = [("sink_bf16", _p), ("dist_r1_bf16", _p), ("dist_r2_bf16", _p), ("talk_bf16", _p), ("gate_per_element", _i), ("chunk", _i)]
 
 
 class VokepelLayerConfig(C.Structure):
@@ -419,8 +424,25 @@ class FofinexConfig(C.Structure):
     ]
 
 
+class LarolornLayerConfig(C.Structure):
+    """struct vmx_larolorn_layer_config (include/vmx.h)."""
+    _fields_ = [
+        ("mixer", _i), ("heads", _i), ("dim", _i), ("vdim", _i), ("scale", _f), ("mask", _i), ("rot", Rotation), ("rot_dim", _i), ("kv_rank", _i),
+        ("kv_heads", _i), ("r_heads", _i), ("r_dim", _i), ("r_vdim", _i), ("decay", C.POINTER(_f)), ("mlp", _i), ("ff", _i), ("limit", _f),
+        ("weights_of", _i),
+    ]
+
+
+class LarolornConfig(C.Structure):
+    """struct vmx_larolorn_config (include/vmx.h)."""
+    _fields_ = [
+        ("vocab", _i), ("width", _i), ("num_layers", _i), ("norm_eps", _f), ("residual_mult", _f), ("logit_scale", _f), ("dtype", _i),
+        ("block_size", _i), ("num_blocks", _i), ("max_tokens", _i), ("max_seqs", _i), ("state_slots", _i),
+    ]
+
+
 # one-family libraries (csrc/Makefile FAMILY=...): the entry points of the other families are absent and stay unbound
-FAMILY_LIBS = ("vokepel", "gezozen", "fofinex")
+FAMILY_LIBS = ("vokepel", "gezozen", "fofinex", "larolorn")
 
 
 def _bind():

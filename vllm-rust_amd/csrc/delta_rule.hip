@@ -595,6 +595,42 @@ __global__ __launch_bounds__(256) void head_rms_gate_kernel(void *__restrict__ y
     }
 }
 
+// The same for wide heads (all of a token's heads normed together, say): a workgroup per (token, head), rows of up to 4096 numbers
+// held in registers between the statistics and the scaling.
+__global__ __launch_bounds__(256) void row_rms_gate_kernel(void *__restrict__ y, int y_f32, const float *__restrict__ o, int64_t ldo,
+                                                            const uint16_t *__restrict__ w, const float *__restrict__ gate, int64_t ldgate,
+                                                            float eps, int heads, int vdim, int gate_silu, int w_per_head) {
+    __shared__ float red[4];
+    constexpr int HELD = 16;
+    const int t = blockIdx.x / heads, h = blockIdx.x % heads, tid = threadIdx.x;
+    const float *src = o + (int64_t)t * ldo + (int64_t)h * vdim;
+    if (gate) gate += (int64_t)t * ldgate + (int64_t)h * vdim;
+    if (w && w_per_head) w += (int64_t)h * vdim;
+    float v[HELD], z[HELD], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < HELD; u++) {
+        const int i = tid + 256 * u;
+        v[u] = i < vdim ? src[i] : 0.f;
+        z[u] = gate && i < vdim ? gate[i] : 0.f;
+    }
+#pragma unroll
+    for (int u = 0; u < HELD; u++) ss = fmaf(v[u], v[u], ss);
+    for (int i = tid + 256 * HELD; i < vdim; i += 256) ss = fmaf(src[i], src[i], ss);
+    const float inv = 1.0f / sqrtf(vmx_block_sum_256(ss, red) / (float)vdim + eps);
+    auto finish = [&](int i, float x, float g) {
+        x *= inv;
+        if (w) x *= vmx_bf16_to_f32(w[i]);
+        if (gate) x *= gate_silu ? silu_f(g) : sigmoid_f(g);
+        const int64_t at = (int64_t)blockIdx.x * vdim + i;
+        if (y_f32) ((float *)y)[at] = x;
+        else ((uint16_t *)y)[at] = vmx_f32_to_bf16(x);
+    };
+#pragma unroll
+    for (int u = 0; u < HELD; u++)
+        if (tid + 256 * u < vdim) finish(tid + 256 * u, v[u], z[u]);
+    for (int i = tid + 256 * HELD; i < vdim; i += 256) finish(i, src[i], gate ? gate[i] : 0.f);
+}
+
 ConvArgs conv_args(const float *x, int64_t ldx, const uint16_t *taps, float *state, float *y, int64_t ldy, const int32_t *positions,
                    const int32_t *seq_ids, const int32_t *seq_starts, const int32_t *state_slots, int tokens, int channels, int n, int group,
                    int unit_groups, int scaled_groups, float unit_eps, float mul) {
@@ -774,6 +810,12 @@ extern "C" int vmx_head_read_out(void *y, int y_dtype, const float *o, int64_t l
     VMX_REQUIRE(!opts->norm || opts->floor, "head_rms_gate: a normaliser comes with its floor");
     VMX_REQUIRE(y_dtype == VMX_F32 || y_dtype == VMX_BF16, "head_rms_gate: f32 or bf16 output");
     if (tokens <= 0) return VMX_OK;
+    if (vdim > 256 && !opts->norm) {
+        hipLaunchKernelGGL(row_rms_gate_kernel, dim3(tokens * heads), dim3(256), 0, vmx_stream(stream), y, y_dtype == VMX_F32, o, ldo, w_bf16, gate, ldgate,
+                           eps, heads, vdim, opts->gate_silu ? 1 : 0, opts->w_per_head ? 1 : 0);
+        VMX_CHECK_LAUNCH("head_rms_gate (wide)");
+        return VMX_OK;
+    }
     hipLaunchKernelGGL(head_rms_gate_kernel, dim3((tokens * heads + 3) / 4), dim3(256), 0, vmx_stream(stream), y, y_dtype == VMX_F32, o, ldo,
                        w_bf16, gate, ldgate, eps, tokens * heads, heads, vdim, opts->gate_silu ? 1 : 0, opts->w_per_head ? 1 : 0, opts->norm,
                        opts->ldnorm, opts->floor, opts->ldfloor, opts->norm_eps);

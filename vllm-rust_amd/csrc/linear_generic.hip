@@ -6,7 +6,8 @@
 //   * gathered activation rows and per-row-block weight matrices (experts of a mixture whose (token, slot) pairs were sorted into
 //     blocks by vmx_moe_align_block_size);
 //   * an optional bf16 bias per output column, then an epilogue: plain store, squared ReLU, tanh-form GELU, accumulate into an
-//     f32 residual stream, multiply by sigmoid(gate), or both of the last two (a gated residual update).
+//     f32 residual stream, multiply by sigmoid(gate), or both of the last two (a gated residual update); a range of output columns
+//     may go through SiLU, so that one product serves readers that want it and readers that do not.
 // Kernels: `linear_mfma_kernel` (64-row tiles for prompts and 64-row expert blocks; a staged 16-row form for shapes the streaming
 // kernel does not take) and `linear_skinny_kernel` (up to 16 rows: decode steps and 16-row expert blocks, weights streamed once)
 // round the activations to bf16 and run v_mfma_f32_16x16x32_bf16; `linear_fma_kernel` multiplies in true f32 on the vector ALU
@@ -29,9 +30,10 @@ __device__ __forceinline__ void linear_store(const VmxLinear &p, int z, int m, i
     } else if (p.epilogue == VMX_EP_GELU_TANH) {
         v = 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
     } else if (p.epilogue == VMX_EP_MUL_SIGMOID || p.epilogue == VMX_EP_ADD_MUL_SIGMOID) {
-        const float g = p.aux[(int64_t)m * p.ldaux + n + z * p.aux_bs];
+        const float g = p.aux[(int64_t)m * p.ldaux + (int64_t)n * p.aux_sn + z * p.aux_bs];
         v *= 1.0f / (1.0f + expf(-g));
     }
+    if (n >= p.silu_begin && n < p.silu_end) v /= 1.0f + expf(-v);
     v *= p.out_scale;
     const int64_t o = (int64_t)m * p.ldc + n + z * p.c_bs;
     if (p.epilogue == VMX_EP_ADD_F32 || p.epilogue == VMX_EP_ADD_MUL_SIGMOID) ((float *)p.C)[o] += v;

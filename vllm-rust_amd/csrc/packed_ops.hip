@@ -1,5 +1,5 @@
 // Kernels that every packed-step executor needs around its mixers and linears: RMS and layer norm of the f32 residual stream (a
-// gain per column or one gain for the row), the norms on both sides of a residual sum in one pass, gated activations, the inverse
+// gain per column or one gain for the row), the norms around a residual sum in one pass, gated activations, the inverse
 // map and the weighted combine of a mixture of experts whose (token, slot) pairs were sorted into expert blocks, greedy ids of f32
 // logits rows, a fill, the step table of a rotary position code.
 #include "vmx_kernels.h"
@@ -70,11 +70,11 @@ __global__ __launch_bounds__(256) void row_norm_f32in_kernel(void *__restrict__ 
     }
 }
 
-// Both norms around a residual sum in one pass over the row: x <- [x +] N(y) * w_post, h = N(x) * w_next (w_next NULL: no h).
-// y[t] is a row of numbers, a row of the embedding table, or the combined result of a mixture of experts.  N as above, centred or
-// not.  A thread keeps HELD groups of VEC neighbouring columns in registers from the first read to the last store, and every load
+// The norms around a residual sum in one pass over the row: x <- [x +] post_mul * N(y) * w_post (w_post NULL: y itself), h = N(x) * w_next
+// (w_next NULL: h = x, or no h).  y[t] is a row of numbers, a row of the embedding table, the combined result of a mixture of experts,
+// or (SIDE) the scaled sum of two branches that each have a norm of their own.  N as above, centred or not.  A thread keeps HELD groups of VEC neighbouring columns in registers from the first read to the last store, and every load
 // that does not depend on a statistic is issued before the first one.  HELD 0: any width, y is formed anew in every pass (at most
-// three) and the new x is read back by the thread that wrote it.
+// three, five with two branches) and the new x is read back by the thread that wrote it.
 template <int VEC> struct SandwichVec;
 template <> struct SandwichVec<4> {
     static __device__ __forceinline__ void ld(const float *p, float *v) {
@@ -99,10 +99,10 @@ template <> struct SandwichVec<1> {
     static __device__ __forceinline__ void st(uint16_t *p, const float *v) { p[0] = vmx_f32_to_bf16(v[0]); }
 };
 
-template <int HELD, int VEC>
+template <int HELD, int VEC, bool SIDE>
 __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a) {
     using V = SandwichVec<VEC>;
-    __shared__ float red[4][4];      // a row per reduction: one barrier each
+    __shared__ float red[8][4];      // a row per reduction: one barrier each
     constexpr int G = HELD ? HELD : 1;
     const int t = blockIdx.x, tid = threadIdx.x, W = a.width;
     float *x = a.x + (int64_t)t * W;
@@ -121,6 +121,7 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a)
     }
     if constexpr (HELD > 0) {
         float y[G][VEC], xv[G][VEC], wp[G][VEC], wn[G][VEC];
+        float sd[SIDE ? G : 1][VEC], wy[SIDE ? G : 1][VEC], ws[SIDE ? G : 1][VEC];
         int col[G];
         bool in[G];
 #pragma unroll
@@ -129,6 +130,9 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a)
             in[u] = col[u] < W;
 #pragma unroll
             for (int e = 0; e < VEC; e++) y[u][e] = xv[u][e] = wp[u][e] = wn[u][e] = 0.f;
+            if constexpr (SIDE)
+#pragma unroll
+                for (int e = 0; e < VEC; e++) sd[u][e] = wy[u][e] = ws[u][e] = 0.f;
         }
 #pragma unroll
         for (int u = 0; u < G; u++)
@@ -136,7 +140,12 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a)
                 if (a.embed) V::ld(erow + col[u], y[u]);
                 else if (!a.pair_rows) V::ld(a.y + (int64_t)t * W + col[u], y[u]);
                 if (a.accumulate) V::ld(x + col[u], xv[u]);
-                V::ld(a.w_post + col[u], wp[u]);
+                if (a.w_post) V::ld(a.w_post + col[u], wp[u]);
+                if constexpr (SIDE) {
+                    V::ld(a.side + (int64_t)t * W + col[u], sd[u]);
+                    V::ld(a.w_y + col[u], wy[u]);
+                    V::ld(a.w_side + col[u], ws[u]);
+                }
                 if (a.w_next) V::ld(a.w_next + col[u], wn[u]);
             }
         if (a.pair_rows && !a.embed) {
@@ -191,13 +200,32 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a)
                 }
             return 1.0f / sqrtf(block_sum(ss, k + 1) * inv_w + a.eps);
         };
-        float mean;
-        float inv = statistics(y, 0, mean);
+        float mean = 0.f, inv = 1.f;
+        if constexpr (SIDE) {
+            float mean_s;
+            const float iy = statistics(y, 4, mean), is = statistics(sd, 6, mean_s);
+#pragma unroll
+            for (int u = 0; u < G; u++)
+#pragma unroll
+                for (int e = 0; e < VEC; e++)   // columns past the row have no gains: 0
+                    y[u][e] = a.side_mul * ((y[u][e] - mean) * iy * wy[u][e] + (sd[u][e] - mean_s) * is * ws[u][e]);
+        }
+        if (a.w_post) inv = statistics(y, 0, mean) * a.post_mul;
+        else mean = 0.f, inv = a.post_mul;
 #pragma unroll
         for (int u = 0; u < G; u++) {
 #pragma unroll
-            for (int e = 0; e < VEC; e++) xv[u][e] = in[u] ? xv[u][e] + (y[u][e] - mean) * inv * wp[u][e] : 0.f;
+            for (int e = 0; e < VEC; e++) xv[u][e] = in[u] ? xv[u][e] + (y[u][e] - mean) * inv * (a.w_post ? wp[u][e] : 1.f) : 0.f;
             if (in[u]) V::st(x + col[u], xv[u]);
+        }
+        if (a.copy_h) {
+#pragma unroll
+            for (int u = 0; u < G; u++)
+                if (in[u]) {
+                    if (a.h_f32) V::st((float *)a.h + (int64_t)t * W + col[u], xv[u]);
+                    else V::st((uint16_t *)a.h + (int64_t)t * W + col[u], xv[u]);
+                }
+            return;
         }
         if (!a.w_next) return;
         inv = statistics(xv, 2, mean);
@@ -232,10 +260,28 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(const VmxSandwich a)
             }
             return 1.0f / sqrtf(block_sum(ss, k + 1) * inv_w + a.eps);
         };
-        float mean;
-        float inv = statistics(y_at, 0, mean);
-        for (int i = tid; i < W; i += 256) x[i] = (a.accumulate ? x[i] : 0.f) + (y_at(i) - mean) * inv * vmx_bf16_to_f32(a.w_post[i]);
-        if (!a.w_next) return;
+        float mean_y = 0.f, mean_s = 0.f, iy = 1.f, is = 1.f;
+        if constexpr (SIDE) {
+            iy = statistics(y_at, 4, mean_y);
+            is = statistics([&](int i) { return a.side[(int64_t)t * W + i]; }, 6, mean_s);
+        }
+        auto branch_at = [&](int i) {   // what goes into the norm after the sublayer
+            if constexpr (SIDE)
+                return a.side_mul * ((y_at(i) - mean_y) * iy * vmx_bf16_to_f32(a.w_y[i]) +
+                                     (a.side[(int64_t)t * W + i] - mean_s) * is * vmx_bf16_to_f32(a.w_side[i]));
+            return y_at(i);
+        };
+        float mean = 0.f, inv = a.post_mul;
+        if (a.w_post) inv = statistics(branch_at, 0, mean) * a.post_mul;
+        for (int i = tid; i < W; i += 256) {
+            const float v = (a.accumulate ? x[i] : 0.f) + (branch_at(i) - mean) * inv * (a.w_post ? vmx_bf16_to_f32(a.w_post[i]) : 1.f);
+            x[i] = v;
+            if (a.copy_h) {
+                if (a.h_f32) ((float *)a.h)[(int64_t)t * W + i] = v;
+                else ((uint16_t *)a.h)[(int64_t)t * W + i] = vmx_f32_to_bf16(v);
+            }
+        }
+        if (!a.w_next || a.copy_h) return;
         inv = statistics([&](int i) { return x[i]; }, 2, mean);
         for (int i = tid; i < W; i += 256) {
             const float v = (x[i] - mean) * inv * vmx_bf16_to_f32(a.w_next[i]);
@@ -399,13 +445,22 @@ __global__ __launch_bounds__(256) void embed_scaled_f32_kernel(float *__restrict
 }
 
 // act[r, j] = f(gu[r, j]) * gu[r, ff + j]: the gated activation between the two products of a feed-forward whose gate and up
-// projections were computed as one product; f = silu or (GELU) the tanh form of gelu
-template <bool GELU> __global__ __launch_bounds__(256) void glu_kernel(void *__restrict__ act, int act_f32, const float *__restrict__ gu, int ff) {
+// projections were computed as one product; f = silu or the tanh form of gelu.  CLAMPED: g = min(gate, limit), u clamped to
+// [-limit, limit], act = g sigmoid(slope g) (u + 1)
+enum GluKind { GLU_SILU, GLU_GELU, GLU_CLAMPED };
+template <GluKind KIND>
+__global__ __launch_bounds__(256) void glu_kernel(void *__restrict__ act, int act_f32, const float *__restrict__ gu, int ff, float slope, float limit) {
     const int64_t r = blockIdx.x;             // rows on x: a prompt's (token, expert) pairs can pass the 65535 of the other axes
     const int j = blockIdx.y * 256 + threadIdx.x;
     if (j >= ff) return;
-    const float g = gu[r * 2 * ff + j], u = gu[r * 2 * ff + ff + j];
-    const float f = GELU ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) : g / (1.0f + expf(-g));
+    float g = gu[r * 2 * ff + j], u = gu[r * 2 * ff + ff + j], f;
+    if constexpr (KIND == GLU_GELU) f = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+    else if constexpr (KIND == GLU_SILU) f = g / (1.0f + expf(-g));
+    else {
+        g = fminf(g, limit);
+        f = g / (1.0f + expf(-slope * g));
+        u = fminf(fmaxf(u, -limit), limit) + 1.0f;
+    }
     const float v = f * u;
     if (act_f32) ((float *)act)[r * ff + j] = v;
     else ((uint16_t *)act)[r * ff + j] = vmx_f32_to_bf16(v);
@@ -465,15 +520,22 @@ int vmx_embed_scaled_f32(float *x, const uint16_t *embed, const int32_t *tokens,
 
 int vmx_glu_silu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st) {
     if (rows <= 0) return VMX_OK;
-    hipLaunchKernelGGL(glu_kernel<false>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff);
+    hipLaunchKernelGGL(glu_kernel<GLU_SILU>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff, 0.f, 0.f);
     VMX_CHECK_LAUNCH("glu silu");
     return VMX_OK;
 }
 
 int vmx_glu_gelu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st) {
     if (rows <= 0) return VMX_OK;
-    hipLaunchKernelGGL(glu_kernel<true>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff);
+    hipLaunchKernelGGL(glu_kernel<GLU_GELU>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff, 0.f, 0.f);
     VMX_CHECK_LAUNCH("glu gelu");
+    return VMX_OK;
+}
+
+int vmx_glu_clamped_rows(void *act, int act_f32, const float *gu, int rows, int ff, float slope, float limit, hipStream_t st) {
+    if (rows <= 0) return VMX_OK;
+    hipLaunchKernelGGL(glu_kernel<GLU_CLAMPED>, dim3(rows, (ff + 255) / 256), dim3(256), 0, st, act, act_f32, gu, ff, slope, limit);
+    VMX_CHECK_LAUNCH("glu clamped");
     return VMX_OK;
 }
 
@@ -493,12 +555,17 @@ int vmx_layer_norm_f32in(void *out, int out_f32, const float *x, const int32_t *
 }
 
 int vmx_sandwich_norm(const VmxSandwich &a, int n, hipStream_t st) {
-    VMX_REQUIRE(a.x && a.w_post && a.width >= 1 && (a.embed ? a.tokens && a.vocab >= 1 : a.y != nullptr), "sandwich norm: null pointer");
-    VMX_REQUIRE(!a.w_next || a.h, "sandwich norm: the next norm needs its output rows");
+    VMX_REQUIRE(a.x && a.width >= 1 && (a.embed ? a.tokens && a.vocab >= 1 : a.y != nullptr), "sandwich norm: null pointer");
+    VMX_REQUIRE((!a.w_next && !a.copy_h) || a.h, "sandwich norm: the next norm (or the copy) needs its output rows");
+    VMX_REQUIRE(!a.side || (a.w_y && a.w_side && !a.embed && !a.pair_rows), "sandwich norm: two branches need their gains and plain rows");
     VMX_REQUIRE(!a.pair_rows || (a.pair_w && a.top >= 1), "sandwich norm: expert results need their weights");
     if (n <= 0) return VMX_OK;
     const bool vec = a.width % 4 == 0;   // every row then starts on a 16-byte (f32) / 8-byte (bf16) boundary
-#define SW(held, v) hipLaunchKernelGGL((sandwich_norm_kernel<held, v>), dim3(n), dim3(256), 0, st, a)
+#define SW(held, v)                                                                                          \
+    do {                                                                                                     \
+        if (a.side) hipLaunchKernelGGL((sandwich_norm_kernel<held, v, true>), dim3(n), dim3(256), 0, st, a); \
+        else hipLaunchKernelGGL((sandwich_norm_kernel<held, v, false>), dim3(n), dim3(256), 0, st, a);       \
+    } while (0)
     if (vec && a.width <= 1024) SW(1, 4);
     else if (vec && a.width <= 2048) SW(2, 4);
     else if (vec && a.width <= 4096) SW(4, 4);

@@ -197,8 +197,10 @@ struct VmxLinear {
     int64_t bias_bs = 0;
     int epilogue = VMX_EP_STORE;       // RELU2: max(v, 0)^2; GELU_TANH; ADD_F32: C += v (f32 C); MUL_SIGMOID: v * sigmoid(aux[m, n]);
                                        // ADD_MUL_SIGMOID: C += v * sigmoid(aux[m, n]) (f32 C)
-    const float *aux = nullptr;
+    const float *aux = nullptr;        // gate numbers: aux[m * ldaux + n * aux_sn + batch * aux_bs] (aux_sn 0: one per row and batch)
     int64_t ldaux = 0;
+    int aux_sn = 1;
+    int silu_begin = 0, silu_end = 0;  // output columns [silu_begin, silu_end) go through z * sigmoid(z) (after the bias)
     float out_scale = 1.0f;            // what is stored or added is this times the epilogue's value (C += out_scale * v)
     int exact = 0;                     // 1: multiply in f32 on the vector ALU even where the matrix cores could take bf16 operands
 };
@@ -236,10 +238,11 @@ int vmx_rms_norm_f32in(void *out, int out_f32, const float *x, const int32_t *ro
                        int n, hipStream_t st);
 // the same with the row's mean taken off first (layer norm, a gain per column)
 int vmx_layer_norm_f32in(void *out, int out_f32, const float *x, const int32_t *rows, const uint16_t *w, int width, float eps, int n, hipStream_t st);
-// Both norms around a residual sum in one pass: x[t] <- (accumulate ? x[t] : 0) + N(y[t]) * w_post, h[t] = N(x[t]) * w_next; N a layer
-// norm (centered) or an RMS norm over `width` columns.  y[t] is, in this order: row tokens[t] of the bf16 table `embed`; the sum
-// over s < top of pair_w[t top + s] * (row pair_rows[t top + s] of y) + sigmoid(shared_gate[t ld]) * shared[t] (shared, its gate:
-// optional); row t of y.
+// The norms around a residual sum in one pass: x[t] <- (accumulate ? x[t] : 0) + post_mul * N(y[t]) * w_post (w_post NULL: y[t] as it
+// is), h[t] = N(x[t]) * w_next, or (copy_h) h[t] = x[t]; N a layer norm (centered) or an RMS norm over `width` columns.  y[t] is, in
+// this order: row tokens[t] of the bf16 table `embed`; the sum over s < top of pair_w[t top + s] * (row pair_rows[t top + s] of y) +
+// sigmoid(shared_gate[t ld]) * shared[t] (shared, its gate: optional); with a side branch, side_mul * (N(y[t]) * w_y + N(side[t]) *
+// w_side); row t of y.
 struct VmxSandwich {
     float *x = nullptr;
     const float *y = nullptr;
@@ -251,8 +254,11 @@ struct VmxSandwich {
     int top = 0;
     const float *shared = nullptr, *shared_gate = nullptr;
     int64_t ld_shared_gate = 0;
-    int accumulate = 1, centered = 1;
-    const uint16_t *w_post = nullptr, *w_next = nullptr;   // w_next NULL: only the sum
+    const float *side = nullptr;
+    const uint16_t *w_y = nullptr, *w_side = nullptr;
+    float side_mul = 1.f, post_mul = 1.f;
+    int accumulate = 1, centered = 1, copy_h = 0;
+    const uint16_t *w_post = nullptr, *w_next = nullptr;   // w_next NULL (and no copy_h): only the sum
     void *h = nullptr;
     int h_f32 = 0, width = 0;
     float eps = 0.f;
@@ -281,6 +287,8 @@ int vmx_embed_scaled_f32(float *x, const uint16_t *embed, const int32_t *tokens,
 int vmx_glu_silu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st);
 // act[r, j] = gelu(gu[r, j]) * gu[r, ff + j], the tanh form of gelu
 int vmx_glu_gelu_rows(void *act, int act_f32, const float *gu, int rows, int ff, hipStream_t st);
+// act[r, j] = g sigmoid(slope g) (u + 1), g = min(gu[r, j], limit), u = gu[r, ff + j] clamped to [-limit, limit]
+int vmx_glu_clamped_rows(void *act, int act_f32, const float *gu, int rows, int ff, float slope, float limit, hipStream_t st);
 // out[t] = [a[t] | b[t]]: two f32 rows of `width` numbers side by side, stored in f32 or bf16
 int vmx_concat2_rows(void *out, int out_f32, const float *a, const float *b, int T, int width, hipStream_t st);
 // x <- cap * tanh(x * scale / cap) over n numbers (cap 0: x * scale)

@@ -1,21 +1,22 @@
 // Grouped-query attention over a paged key/value cache for packed steps, with the score shaping some decoder families use:
 //   s_j = (q . k_j) * scale * temp[h];  s_j <- cap * tanh(s_j / cap) (cap > 0);  p = softmax over the visible j;  o = sum_j p_j v_j
 // Position i of a sequence sees j <= i when i - j < window (window 0: every earlier key) or j < keep_first (the first tokens of
-// the sequence stay visible after the window has passed them).  No rotation: positions only decide visibility.  Query head h
+// the sequence stay visible after the window has passed them).  With chunks of c positions, counted from the sequence's position 0,
+// i also sees only keys of its own chunk (or of the kept first tokens).  No rotation: positions only decide visibility.  Query head h
 // reads key/value head h / (heads / kv_heads); key and value widths may differ.  The head's output may be multiplied by
 // sigmoid(gate[t, h]) (one number per token and head, or one per output element) before it is stored.
 // Extras (vmx_window_attention_ex), each optional: a learned sink per head in the softmax denominator (exp(sink), no key, no value);
 // a logarithmic distance penalty s_j -= r1[h] * ln(1 + r2[h] * (i - j)) after the soft cap; mixing of the heads' scores,
 // s_h <- sum_g talk[h, g] s_g at every visible key, before the softmax (all heads of a token then run in one workgroup).
 // vmx_qk_prepare_cache_write readies a step's projected rows: whole-row RMS norms of q and k, pair rotation, cache write;
-// vmx_qk_prepare_ex does the same head by head (norms over each head with gains shared by the heads, rotation of neighbouring
-// coordinates or of the two halves of the rotated run, scaled cos / sin, constant multipliers, keys to plain rows for a mixer
-// that keeps no cache).
+// vmx_qk_prepare_ex has its options open (norms over whole rows, or over each head with gains shared by the heads; rotation of
+// neighbouring coordinates or of the two halves of the rotated run, scaled cos / sin, constant multipliers, keys to plain rows for
+// a mixer that keeps no cache).
 //
 // Keys and values live in two caches of rows [kv_heads * dim] / [kv_heads * vdim], bf16 or f32; a step writes its new rows first
 // (vmx_kv_cache_write_f32) and prompts, prompt portions and decode tokens then run the SAME kernel over the cache, so a row's
 // result does not depend on how its prompt was cut or on what else is in the step.  Scores, softmax and the weighted sum are f32.
-// The visible keys of a row are two runs, [0, min(keep_first, lo)) and [lo, i] with lo = max(0, i - window + 1).  Two kernels:
+// The visible keys of a row are two runs, [0, min(keep_first, lo)) and [lo, i] with lo = first_key(i).  Two kernels:
 // the vector form (any sizes, f32 or bf16 cache: a wave owns one (token, head) row and walks its keys 64 at a time, lane l scores
 // key l of the tile, then every lane sums its value columns) and the matrix-core form below for bf16 caches.
 #include "vmx_kernels.h"
@@ -70,6 +71,12 @@ struct WinAttn {
     float *ws;                   // [tokens, heads, parts, vdim + 2]: unnormalised sums, running maximum, denominator
     const uint16_t *sink, *r1, *r2, *talk;   // extras, each NULL when absent
     int gate_elem;               // 1: gate rows hold heads * vdim numbers
+    int chunk;                   // > 0: only keys of the query's own chunk of positions
+    // first key of the run that ends at position i
+    __device__ __forceinline__ int first_key(int i) const {
+        const int lo = window > 0 ? max(0, i - window + 1) : 0;
+        return chunk > 0 ? max(lo, i - i % chunk) : lo;
+    }
 };
 
 __device__ __forceinline__ float sigmoid_f32(float x) { return 1.0f / (1.0f + expf(-x)); }
@@ -81,62 +88,6 @@ __device__ __forceinline__ void add_sink(float sink, float &m, float &den, float
     f = expf(m - mn);
     den = den * f + expf(sink - mn);
     m = mn;
-}
-
-// q_out[t] / key row of token t: optional whole-row RMS norm, optional pair rotation inside every head, keys and values to the cache
-__global__ __launch_bounds__(256) void qk_prepare_kernel(float *__restrict__ q_out, const float *__restrict__ q, int64_t ldq, int qw,
-                                                          const float *__restrict__ k, int64_t ldk, int kw, const float *__restrict__ v,
-                                                          int64_t ldv, int vw, const uint16_t *__restrict__ qn, const uint16_t *__restrict__ kn,
-                                                          float eps, const float *__restrict__ inv_freq, int rot_dims, int head_dim,
-                                                          const int32_t *__restrict__ positions, const int32_t *__restrict__ slots,
-                                                          void *__restrict__ kc, void *__restrict__ vc, int f32) {
-    __shared__ float red[4];
-    const int t = blockIdx.x, tid = threadIdx.x;
-    const float *qr = q + (int64_t)t * ldq, *kr = k + (int64_t)t * ldk, *vr = v + (int64_t)t * ldv;
-    float qinv = 1.0f, kinv = 1.0f;
-    if (qn) {
-        float ss = 0.f;
-        for (int i = tid; i < qw; i += 256) ss += qr[i] * qr[i];
-        ss = vmx_block_sum_256(ss, red);
-        qinv = 1.0f / sqrtf(ss / (float)qw + eps);
-        __syncthreads();
-    }
-    if (kn) {
-        float ss = 0.f;
-        for (int i = tid; i < kw; i += 256) ss += kr[i] * kr[i];
-        ss = vmx_block_sum_256(ss, red);
-        kinv = 1.0f / sqrtf(ss / (float)kw + eps);
-    }
-    const float pos = (float)positions[t];
-    const int64_t slot = slots[t];
-    const bool rot = inv_freq && rot_dims > 0;
-    for (int i = tid; i < qw + kw; i += 256) {
-        const bool isq = i < qw;
-        const int e = isq ? i : i - qw;
-        const float *src = isq ? qr : kr;
-        const uint16_t *w = isq ? qn : kn;
-        const float inv = isq ? qinv : kinv;
-        float x = src[e] * inv;
-        if (w) x *= vmx_bf16_to_f32(w[e]);
-        const int c = e % head_dim;
-        if (rot && c < rot_dims) {
-            float y = src[e ^ 1] * inv;   // the pair's other coordinate (rot_dims and head_dim are even)
-            if (w) y *= vmx_bf16_to_f32(w[e ^ 1]);
-            float sn, cs;
-            sincosf(pos * inv_freq[c >> 1], &sn, &cs);
-            x = (c & 1) ? x * cs + y * sn : x * cs - y * sn;
-        }
-        if (isq) q_out[(int64_t)t * qw + e] = x;
-        else if (slot >= 0) {
-            if (f32) ((float *)kc)[slot * kw + e] = x;
-            else ((uint16_t *)kc)[slot * kw + e] = vmx_f32_to_bf16(x);
-        }
-    }
-    if (slot >= 0)
-        for (int i = tid; i < vw; i += 256) {
-            if (f32) ((float *)vc)[slot * vw + i] = vr[i];
-            else ((uint16_t *)vc)[slot * vw + i] = vmx_f32_to_bf16(vr[i]);
-        }
 }
 
 struct QkPrep {
@@ -155,6 +106,65 @@ struct QkPrep {
     float *k_out;
     int64_t ldk_out;
 };
+
+// One workgroup per token: optional RMS norms over the WHOLE query and key rows, optional rotation of every head's first rot_dims
+// coordinates (pairs as in the form below; the token's angles are computed once, in LDS), constant multipliers; queries to q_out,
+// keys to the cache row slots[t] or to k_out[t], values to the cache.
+__global__ __launch_bounds__(256) void qk_prepare_kernel(const QkPrep a) {
+    __shared__ float red[4];
+    __shared__ float2 turn[128];
+    const int t = blockIdx.x, tid = threadIdx.x, hd = a.head_dim, half = a.rot_dims >> 1;
+    const float *qr = a.q + (int64_t)t * a.ldq, *kr = a.k + (int64_t)t * a.ldk;
+    const float pos = (float)a.positions[t];
+    auto angle = [&](int i) {
+        float sn, cs;
+        sincosf(pos * a.inv_freq[i], &sn, &cs);
+        return make_float2(cs * a.rot_mul, sn * a.rot_mul);
+    };
+    for (int i = tid; i < min(half, 128); i += 256) turn[i] = angle(i);
+    auto row_scale = [&](const float *row, int n) {
+        float ss = 0.f;
+        for (int i = tid; i < n; i += 256) ss += row[i] * row[i];
+        ss = vmx_block_sum_256(ss, red);
+        return 1.0f / sqrtf(ss / (float)n + a.eps);
+    };
+    const float qinv = a.qn ? row_scale(qr, a.qw) : 1.0f;
+    __syncthreads();   // the angles are there, and the first sum has been read
+    const float kinv = a.kn ? row_scale(kr, a.kw) : 1.0f;
+    const int64_t slot = a.slots ? a.slots[t] : -1;
+    for (int i = tid; i < a.qw + a.kw; i += 256) {
+        const bool isq = i < a.qw;
+        const int e = isq ? i : i - a.qw, c = e % hd;
+        const float *src = isq ? qr : kr;
+        const uint16_t *w = isq ? a.qn : a.kn;
+        const float inv = isq ? qinv : kinv;
+        float x = src[e] * inv;
+        if (w) x *= vmx_bf16_to_f32(w[e]);
+        if (c < a.rot_dims) {
+            const bool second = a.rot_halves ? c >= half : (c & 1);
+            const int pe = a.rot_halves ? (second ? e - half : e + half) : (second ? e - 1 : e + 1);
+            const int fi = a.rot_halves ? (second ? c - half : c) : (c >> 1);
+            float y = src[pe] * inv;   // the pair's other coordinate
+            if (w) y *= vmx_bf16_to_f32(w[pe]);
+            const float2 cs = fi < 128 ? turn[fi] : angle(fi);
+            x = second ? x * cs.x + y * cs.y : x * cs.x - y * cs.y;
+        }
+        x *= isq ? a.q_mul : a.k_mul;
+        if (isq) a.q_out[(int64_t)t * a.qw + e] = x;
+        else if (a.k_out) a.k_out[(int64_t)t * a.ldk_out + e] = x;
+        else if (slot >= 0) {
+            if (a.f32) ((float *)a.kc)[slot * a.kw + e] = x;
+            else ((uint16_t *)a.kc)[slot * a.kw + e] = vmx_f32_to_bf16(x);
+        }
+    }
+    if (a.v && a.vc && slot >= 0) {
+        const float *vr = a.v + (int64_t)t * a.ldv;
+        for (int i = tid; i < a.vw; i += 256) {
+            if (a.f32) ((float *)a.vc)[slot * a.vw + i] = vr[i];
+            else ((uint16_t *)a.vc)[slot * a.vw + i] = vmx_f32_to_bf16(vr[i]);
+        }
+    }
+}
 
 // One wave per (token, query or key head): optional RMS norm over the head (gains of head_dim numbers, the same for every head),
 // optional rotation of the head's first rot_dims coordinates, a constant multiplier; queries to q_out, keys to the cache row
@@ -229,7 +239,7 @@ __global__ __launch_bounds__(256) void window_attn_wave_kernel(const WinAttn p) 
     const float qmul = p.scale * (p.temp ? vmx_bf16_to_f32(p.temp[h]) : 1.0f);
     for (int i = lane; i < D; i += 64) qs[wave][i] = p.q[(int64_t)t * p.ldq + (int64_t)h * D + i] * qmul;
     __builtin_amdgcn_wave_barrier();
-    const int lo = p.window > 0 ? max(0, pos - p.window + 1) : 0;
+    const int lo = p.first_key(pos);
     const int na = min(p.keep_first, lo), n = na + (pos - lo + 1);
     const float inv_cap = p.softcap > 0.f ? 1.0f / p.softcap : 0.f;
     float m = -FLT_MAX, den = 0.f, acc[VPL];
@@ -307,7 +317,7 @@ __global__ __launch_bounds__(512) void window_attn_talk_kernel(const WinAttn p) 
         qs[i] = p.q[(int64_t)t * p.ldq + i] * p.scale * (p.temp ? vmx_bf16_to_f32(p.temp[i / D]) : 1.0f);
     for (int i = threadIdx.x; i < H * H; i += blockDim.x) tk[i] = vmx_bf16_to_f32(p.talk[i]);
     __syncthreads();
-    const int lo = p.window > 0 ? max(0, pos - p.window + 1) : 0;
+    const int lo = p.first_key(pos);
     const int na = min(p.keep_first, lo), n = na + (pos - lo + 1);
     const float inv_cap = p.softcap > 0.f ? 1.0f / p.softcap : 0.f;
     float m[HPW], den[HPW], acc[HPW][VPL];
@@ -428,11 +438,11 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(const WinAttn p) 
     const int D = p.dim, V = p.vdim;
     const int64_t kw = (int64_t)p.kv_heads * D, vw = (int64_t)p.kv_heads * V;
     const int i0 = p.positions[r0], i1 = i0 + nrows - 1;
-    const int lo = p.window > 0 ? max(0, i0 - p.window + 1) : 0;
+    const int lo = p.first_key(i0);
     const int na = min(p.keep_first, lo), nk = na + (i1 - lo + 1);
     const int32_t *bt = p.block_tables + (int64_t)p.seq_ids[r0] * p.max_blocks;
     const uint16_t *kc = (const uint16_t *)p.kc, *vc = (const uint16_t *)p.vc;
-    const int qrow = 16 * sub + fl, qi = i0 + qrow;
+    const int qrow = 16 * sub + fl, qi = i0 + qrow, qlo = p.first_key(qi);
     const bool qlive = active && qrow < nrows;
     uint4 qf[DS];
 #pragma unroll
@@ -531,7 +541,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(const WinAttn p) 
                 for (int r = 0; r < 4; r++) {
                     const int idx = kb + 16 * kt + 4 * fg + r;
                     const int j = idx < na ? idx : lo + (idx - na);
-                    const bool vis = qlive && idx < kb1 && j <= qi && (p.window == 0 || qi - j < p.window || j < p.keep_first);
+                    const bool vis = qlive && idx < kb1 && j <= qi && (j >= qlo || j < p.keep_first);
                     float x = acc[r] * smul;
                     if (p.softcap > 0.f) x = p.softcap * tanh_fast(x * inv_cap);
                     if (p.r1) x -= dr1 * __logf(1.0f + dr2 * (float)max(qi - j, 0));
@@ -661,11 +671,11 @@ __global__ __launch_bounds__(TM_NT) void talk_attn_mfma_kernel(const WinAttn p) 
     if (nrows <= 0) return;   // the same for the whole workgroup
     const int64_t kw = (int64_t)G * D, vw = (int64_t)G * V;
     const int i0 = p.positions[r0], i1 = i0 + nrows - 1;
-    const int lo = p.window > 0 ? max(0, i0 - p.window + 1) : 0;
+    const int lo = p.first_key(i0);
     const int na = min(p.keep_first, lo), nk = na + (i1 - lo + 1);
     const int32_t *bt = p.block_tables + (int64_t)p.seq_ids[r0] * p.max_blocks;
     const uint16_t *kc = (const uint16_t *)p.kc, *vc = (const uint16_t *)p.vc;
-    const int qi = i0 + fl;
+    const int qi = i0 + fl, qlo = p.first_key(qi);
     const bool qlive = fl < nrows;
     uint4 qf[HPW][DS];
     float smul[HPW], dr1[HPW], dr2[HPW];
@@ -824,7 +834,7 @@ __global__ __launch_bounds__(TM_NT) void talk_attn_mfma_kernel(const WinAttn p) 
                     for (int r = 0; r < 4; r++) {
                         const int idx = kb + 16 * kt + 4 * fg + r;
                         const int j = idx < na ? idx : lo + (idx - na);
-                        const bool vis = qlive && idx < kb1 && j <= qi && (p.window == 0 || qi - j < p.window || j < p.keep_first);
+                        const bool vis = qlive && idx < kb1 && j <= qi && (j >= qlo || j < p.keep_first);
                         sc[kt][r] = vis ? mx[r] : -FLT_MAX;
                         tmax = fmaxf(tmax, sc[kt][r]);
                     }
@@ -995,9 +1005,9 @@ extern "C" int vmx_qk_prepare_cache_write(float *q_out, const float *q, int64_t 
     VMX_REQUIRE(!rot || (rot_dims % 2 == 0 && rot_dims <= head_dim && head_dim % 2 == 0),
                 "qk_prepare: %d rotated coordinates in heads of %d (pairs inside a head of even size)", rot_dims, head_dim);
     if (tokens <= 0) return VMX_OK;
-    hipLaunchKernelGGL(qk_prepare_kernel, dim3(tokens), dim3(256), 0, vmx_stream(stream), q_out, q, ldq, q_width, k, ldk, k_width, v, ldv, v_width,
-                       q_norm_bf16, k_norm_bf16, eps, inv_freq, rot ? rot_dims : 0, head_dim, positions, slots, k_cache, v_cache,
-                       cache_dtype == VMX_F32);
+    const QkPrep a{q_out, q, k, v, ldq, ldk, ldv, q_width, k_width, v_width, q_norm_bf16, k_norm_bf16, eps, inv_freq, rot ? rot_dims : 0, head_dim,
+                   positions, slots, k_cache, v_cache, cache_dtype == VMX_F32, 0, 1.0f, 1.0f, 1.0f, nullptr, 0};
+    hipLaunchKernelGGL(qk_prepare_kernel, dim3(tokens), dim3(256), 0, vmx_stream(stream), a);
     VMX_CHECK_LAUNCH("qk_prepare");
     return VMX_OK;
 }
@@ -1017,7 +1027,6 @@ extern "C" int vmx_qk_prepare_ex(float *q_out, const float *q, int64_t ldq, int 
     VMX_REQUIRE(q_width >= 1 && k_width >= 1 && ldq >= q_width && ldk >= k_width && (!cached || (v_width >= 1 && ldv >= v_width)),
                 "qk_prepare_ex: bad row widths");
     VMX_REQUIRE(head_dim >= 1 && q_width % head_dim == 0 && k_width % head_dim == 0, "qk_prepare_ex: rows are not whole heads of %d", head_dim);
-    VMX_REQUIRE(o.norm_per_head || (!q_norm_bf16 && !k_norm_bf16), "qk_prepare_ex: whole-row norms are vmx_qk_prepare_cache_write's");
     const bool rot = inv_freq && rot_dims > 0;
     VMX_REQUIRE(!rot || (rot_dims % 2 == 0 && rot_dims <= head_dim && (o.rot_halves || head_dim % 2 == 0)),
                 "qk_prepare_ex: %d rotated coordinates in heads of %d", rot_dims, head_dim);
@@ -1026,6 +1035,11 @@ extern "C" int vmx_qk_prepare_ex(float *q_out, const float *q, int64_t ldq, int 
                    rot ? rot_dims : 0, head_dim, positions, cached ? slots : nullptr, cached ? k_cache : nullptr, cached ? v_cache : nullptr,
                    cache_dtype == VMX_F32, o.rot_halves ? 1 : 0, o.rot_mul != 0.f ? o.rot_mul : 1.0f, o.q_mul != 0.f ? o.q_mul : 1.0f,
                    o.k_mul != 0.f ? o.k_mul : 1.0f, o.k_out, o.ldk_out};
+    if (!o.norm_per_head && (q_norm_bf16 || k_norm_bf16)) {
+        hipLaunchKernelGGL(qk_prepare_kernel, dim3(tokens), dim3(256), 0, vmx_stream(stream), a);
+        VMX_CHECK_LAUNCH("qk_prepare_ex (whole rows)");
+        return VMX_OK;
+    }
     const int heads = (q_width + k_width) / head_dim;
     hipLaunchKernelGGL(qk_prepare_heads_kernel, dim3(tokens, (heads + 3) / 4), dim3(256), 0, vmx_stream(stream), a);
     VMX_CHECK_LAUNCH("qk_prepare_ex");
@@ -1056,10 +1070,12 @@ extern "C" int vmx_window_attention_ex(void *out, int out_dtype, const float *q,
                 heads, kv_heads);
     VMX_REQUIRE(dim >= 1 && dim <= WA_MAX_DIM && vdim >= 1 && vdim <= 256, "window_attention: head sizes %d / %d outside 1..256", dim, vdim);
     VMX_REQUIRE(window >= 0 && keep_first >= 0 && block_size >= 1 && max_blocks_per_seq >= 1 && softcap >= 0.f, "window_attention: bad arguments");
-    const vmx_window_attn_extras none = {nullptr, nullptr, nullptr, nullptr, 0};
+    const vmx_window_attn_extras none = {};
     const vmx_window_attn_extras &ex = extras ? *extras : none;
     VMX_REQUIRE(ldq >= (int64_t)heads * dim && (!gate || ldgate >= (ex.gate_per_element ? (int64_t)heads * vdim : heads)),
                 "window_attention: bad row strides");
+    VMX_REQUIRE(ex.chunk >= 0, "window_attention: bad chunk size %d", ex.chunk);
+    const int span = ex.chunk > 0 && (window == 0 || ex.chunk < window) ? ex.chunk : window;   // most keys a row sees besides the kept ones (0: no bound)
     VMX_REQUIRE(!ex.dist_r1_bf16 == !ex.dist_r2_bf16, "window_attention: the distance penalty needs both of its numbers per head");
     VMX_REQUIRE(!ex.talk_bf16 || (heads <= TALK_MAX_HEADS && heads * dim <= TALK_MAX_QS),
                 "window_attention: mixed heads take at most %d heads and %d query numbers per token", TALK_MAX_HEADS, TALK_MAX_QS);
@@ -1067,7 +1083,7 @@ extern "C" int vmx_window_attention_ex(void *out, int out_dtype, const float *q,
     WinAttn p{out, out_dtype == VMX_F32, q, ldq, k_cache, v_cache, block_tables, seq_ids, positions, max_blocks_per_seq, head_temp_bf16,
               gate, ldgate, scale, softcap, window, keep_first, tokens, heads, kv_heads, dim, vdim, block_size, seq_starts, num_seqs,
               (block_size & (block_size - 1)) == 0 ? __builtin_ctz(block_size) : -1, 1, (float *)workspace,
-              ex.sink_bf16, ex.dist_r1_bf16, ex.dist_r2_bf16, ex.talk_bf16, ex.gate_per_element ? 1 : 0};
+              ex.sink_bf16, ex.dist_r1_bf16, ex.dist_r2_bf16, ex.talk_bf16, ex.gate_per_element ? 1 : 0, ex.chunk};
     hipStream_t st = vmx_stream(stream);
     const bool f32 = cache_dtype == VMX_F32;
     if (p.talk && !f32 && seq_starts && num_seqs >= 1 && dim % 8 == 0 && vdim % 8 == 0 && dim <= 256 && vdim <= 128 && ldq % 4 == 0 &&
@@ -1082,7 +1098,7 @@ extern "C" int vmx_window_attention_ex(void *out, int out_dtype, const float *q,
             const int runs = tokens / 16 + num_seqs;
             if (workspace && runs < 128) {
                 int parts = 256 / runs < 32 ? 256 / runs : 32;   // one workgroup holds all heads: a run has few workgroups to begin with
-                if (window > 0) parts = std::min(parts, (window + keep_first + 16 + TM_KT - 1) / TM_KT);
+                if (span > 0) parts = std::min(parts, (span + keep_first + 16 + TM_KT - 1) / TM_KT);
                 parts = std::min<size_t>(parts, workspace_bytes / ((size_t)tokens * heads * (vdim + 2) * 4));
                 if (parts > 1) p.parts = parts;
             }
@@ -1133,7 +1149,7 @@ extern "C" int vmx_window_attention_ex(void *out, int out_dtype, const float *q,
         const int base = runs * kv_heads * ((qpk + 3) / 4);
         if (workspace && base < 128) {   // few workgroups: deal each run's key tiles to several
             int parts = 256 / base < 16 ? 256 / base : 16;
-            if (window > 0) parts = std::min(parts, (window + keep_first + rt + 63) / 64);
+            if (span > 0) parts = std::min(parts, (span + keep_first + rt + 63) / 64);
             parts = std::min<size_t>(parts, workspace_bytes / ((size_t)tokens * heads * (vdim + 2) * 4));
             if (parts > 1) p.parts = parts;
         }
