@@ -62,11 +62,11 @@ class LarolornLayerSpec:
         s.mask = int((a.get("mask") or {}).get("size") or 0)
         s.rot = RotationSpec.from_config(a.get("rot"))
         if kind == "latent_attention":
-            s.rot_dim, s.kv_rank, s.kv_heads = int(a["rot_dim"]), int(a["kv_rank"]), s.heads
+            s.rot_dim, s.kv_rank = int(a["rot_dim"]), int(a["kv_rank"])
             s.scale = float(a.get("scale", 1.0 / math.sqrt(s.dim + s.rot_dim)))
         else:
             r = m["right"]
-            s.rot_dim, s.kv_rank, s.kv_heads = 0, 0, int(a.get("kv_heads", s.heads))
+            s.kv_heads = int(a.get("kv_heads", s.heads))
             s.scale = float(a.get("scale", 1.0 / math.sqrt(s.dim)))
             s.r_heads, s.r_dim, s.r_vdim = int(r["heads"]), int(r["dim"]), int(r.get("vdim", r["dim"]))
             s.decay = tuple(float(d) for d in r["decay"])
