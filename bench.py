@@ -1111,6 +1111,91 @@ def fofinex_workload(prompt, steps, warmup, sizes=("1k", "2k"), batches=(1, 16),
             "data": "synthetic", "prompt": prompt, "sizes": out}
 
 
+LAROLORN_SIZES = {
+    # name: (width, latent heads, dim, rot_dim, vdim, kv_rank, window, attention heads, kv_heads, dim, chunk, memory heads, memory key / value size,
+    #        dense ff, vocab)
+    "1k": (1024, 8, 64, 32, 64, 256, 4096, 8, 2, 128, 4096, 8, 128, 3072, 32000),
+    "2k": (2048, 16, 128, 64, 128, 512, 4096, 16, 4, 128, 4096, 16, 128, 6144, 32000),
+}
+
+
+def larolorn_workload(prompt, steps, warmup, sizes=("1k", "2k"), batches=(1, 16), comparator=True, main=True):
+    """Larolorn (results normed before the sum; windowed latent attention with head gates; chunked sink attention beside a memory with
+    constant decays; clamped gated feed-forwards; bf16 weights) at layer sizes of real models, beside the closest existing models at
+    equal size: Fofinex (latent attention, matrix memory, gated dense feed-forwards) and, for the attention beside a memory, Gezozen
+    (windowed attention beside retention, without feed-forwards).  Larolorn: latent attention + dense, two-sided + dense, twice over;
+    Fofinex: latent attention + dense, memory + dense, twice over; Gezozen: attention | retention four times.  Prompt pass: tokens/s of
+    one `prompt`-token sequence; decode: aggregate tok/s of B sequences at context `prompt`, one hipGraph per step.  main=False times
+    the comparators alone (kernel traces)."""
+    from vllm_rust_amd.fofinex import FofinexForCausalLM, FofinexLayerSpec, FofinexSpec
+    from vllm_rust_amd.fofinex import synthetic_weights as fofinex_weights
+    from vllm_rust_amd.gezozen import GezozenForCausalLM, GezozenLayerSpec, GezozenSpec
+    from vllm_rust_amd.gezozen import synthetic_weights as gezozen_weights
+    from vllm_rust_amd.larolorn import LarolornForCausalLM, LarolornLayerSpec, LarolornSpec, synthetic_weights
+    from vllm_rust_amd.rotation import RotationSpec
+    out = {}
+    dev = torch.device("cuda", torch.cuda.current_device())
+    side = torch.cuda.Stream(device=dev)
+    BM = max(batches)
+    per_seq = (prompt + warmup + steps + 8 + 15) // 16 + 1
+
+    def timed(cls, spec, weights, V):
+        model = cls(spec, "bfloat16", block_size=16, num_blocks=per_seq * BM, max_tokens=max(prompt, BM), max_seqs=BM)
+        model.load_state(weights(spec, 3, device=dev))
+        t = _packed_times(model, V, prompt, batches, warmup, steps, side, dev, True)
+        model.close()
+        return t
+
+    def lines(t, macs, fixed, per_batch):
+        """macs: multiply-adds per prompt token; fixed: bytes a decode step reads whatever B; per_batch(B): the rest."""
+        r = {"prefill": {"tokens": prompt, "ms": round(t["prefill"] * 1e3, 3), "tok_s": round(prompt / t["prefill"], 1),
+                         "TFLOP_s": round(2.0 * prompt * macs / t["prefill"] / 1e12, 2)}}
+        for B in batches:
+            r[f"decode_b{B}"] = {"tok_s": round(B / t[B], 1), "ms_per_step": round(t[B] * 1e3, 4),
+                                 "GBps_algorithmic": round((fixed + per_batch(B)) / t[B] / 1e9, 1)}
+        return r
+    for name in sizes:
+        W, LH, LD, rd, lv, R, win, H, G, D, chunk, MH, MD, ff, V = LAROLORN_SIZES[name]
+        decay = tuple(1.0 - 2.0 ** (-5 - 5 * i / max(MH - 1, 1)) for i in range(MH))
+        seen = lambda size: min(size, prompt / 2) if size >= prompt else size / 2      # mean keys of a row   # noqa: E731
+        kept = lambda size: min(size, prompt + 1)                                       # keys a decode row reads   # noqa: E731
+        lat_lin = W * (LH * (LD + rd) + R + rd + LH) + LH * LD * R + LH * lv * R + LH * lv * W
+        lat_att, two_att, mem = LH * (2 * R + rd), H * 2 * D, MH * 3 * MD * MD
+        two_lin = W * (H * D + 2 * G * D + 4 * MH * MD) + H * D * W + MH * MD * W
+        dense, head = 3 * ff * W, V * W
+        out[name] = {}
+        if main:
+            lat = LarolornLayerSpec(mixer="latent_attention", heads=LH, dim=LD, rot_dim=rd, vdim=lv, kv_rank=R, scale=1.0 / math.sqrt(LD + rd), mask=win,
+                                    rot=RotationSpec(rd, 1e5), mlp="dense", ff=ff, limit=7.0)
+            two = LarolornLayerSpec(mixer="parallel", heads=H, kv_heads=G, dim=D, vdim=D, scale=1.0 / math.sqrt(D), mask=chunk, rot=RotationSpec(D, 1e5),
+                                    r_heads=MH, r_dim=MD, r_vdim=MD, decay=decay, mlp="dense", ff=ff, limit=7.0)
+            spec = LarolornSpec(vocab=V, width=W, layers=[lat, two, lat, two], residual_mult=0.5)
+            lin = 2 * (lat_lin + two_lin) + 4 * dense
+            t = timed(LarolornForCausalLM, spec, synthetic_weights, V)
+            out[name]["larolorn"] = lines(t, lin + 2 * (lat_att * seen(win) + two_att * seen(chunk) + mem) + head / prompt, 2 * (lin + head),
+                                          lambda B: 2 * 2 * B * (kept(win) * (R + rd) + kept(chunk) * 2 * G * D) + 2 * 2 * B * MH * MD * MD * 4)
+        if comparator:
+            Q = 3 * W // 8
+            fl = FofinexLayerSpec(mixer="latent_attention", heads=LH, dim=LD, rot_dim=rd, vdim=lv, kv_rank=R, q_rank=Q, scale=1.0 / math.sqrt(LD + rd),
+                                  rot=RotationSpec(rd, 1e5), mlp="dense", ff=ff)
+            fm = FofinexLayerSpec(mixer="mlstm", heads=MH, dim=MD, vdim=MD, gate_cap=15.0, mlp="dense", ff=ff)
+            flin = 2 * (lat_lin - W * (LH * (LD + rd) + LH) + Q * (W + LH * (LD + rd))) + 2 * (W * (4 * MH * MD + 2 * MH) + MH * MD * W) + 4 * dense
+            t = timed(FofinexForCausalLM, FofinexSpec(vocab=V, width=W, layers=[fl, fm, fl, fm]), fofinex_weights, V)
+            out[name]["fofinex"] = lines(t, flin + 2 * (lat_att * prompt / 2 + mem) + head / prompt, 2 * (flin + head),
+                                         lambda B: 2 * 2 * B * (prompt + 1) * (R + rd) + 2 * 2 * B * MH * MD * (MD + 1) * 4)
+            gl = GezozenLayerSpec(mixer="parallel_2", heads=H, kv_heads=G, dim=D, vdim=D, scale=1.0 / math.sqrt(D), window=chunk, rot=RotationSpec(D, 1e5),
+                                  r_heads=MH, r_dim=MD, r_vdim=MD, decay=decay, r_rot=RotationSpec(MD, 1e4), mlp=None)
+            glin = 4 * (two_lin + W * W)
+            t = timed(GezozenForCausalLM, GezozenSpec(vocab=V, width=W, layers=[gl] * 4, norm_groups=1, postln_alpha=2.0), gezozen_weights, V)
+            out[name]["gezozen"] = lines(t, glin + 4 * (two_att * seen(chunk) + mem) + head / prompt, 2 * (glin + head),
+                                         lambda B: 2 * 4 * B * kept(chunk) * 2 * G * D + 2 * 4 * B * MH * MD * MD * 4)
+        out[name]["config"] = {"width": W, "layers": ["latent_attention+dense", "parallel+dense"] * 2, "latent_heads": LH, "latent_dim": LD, "rot_dim": rd,
+                               "latent_vdim": lv, "kv_rank": R, "window": win, "heads": H, "kv_heads": G, "dim": D, "chunk": chunk, "memory_heads": MH,
+                               "memory_dim": MD, "ff": ff, "vocab": V, "fofinex": ["latent_attention+dense", "mlstm+dense"] * 2, "gezozen": ["parallel_2"] * 4}
+    return {"metric": "Larolorn prompt and decode throughput beside Fofinex and Gezozen at equal size", "unit": "tok/s", "dtype": "bf16",
+            "data": "synthetic", "prompt": prompt, "sizes": out}
+
+
 def plan_job(gpus, world, replicas_flag, weights, local_ranks):
     """What a launch of this script measures -- pure argument logic, no device.  N = 1: the single-GPU job.  N > 1 (one process
     per GPU under torch.distributed.run): ONE model tensor-parallel over the N ranks (BASELINE.json's metric is the TP curve at
@@ -1268,10 +1353,10 @@ def main():
     ap.add_argument("--no-secondary", action="store_true", help="skip the secondary measurements (other models at N = 1, replicas at N > 1)")
     ap.add_argument("--no-moe", action="store_true", help="skip the Mixtral-8x7B-shaped fused-MoE secondary measurement")
     ap.add_argument("--no-comparator", action="store_true",
-                    help="--workload vokepel / gezozen / fofinex: time that executor alone (kernel traces of one model)")
-    ap.add_argument("--comparator-only", action="store_true", help="--workload gezozen / fofinex: time the comparators alone (kernel traces)")
-    ap.add_argument("--sizes", default="1k,2k", help="--workload vokepel / gezozen / fofinex: which of its sizes to run")
-    ap.add_argument("--workload", choices=["all", "qwen3", "gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen", "fofinex"], default="all",
+                    help="--workload vokepel / gezozen / fofinex / larolorn: time that executor alone (kernel traces of one model)")
+    ap.add_argument("--comparator-only", action="store_true", help="--workload gezozen / fofinex / larolorn: time the comparators alone (kernel traces)")
+    ap.add_argument("--sizes", default="1k,2k", help="--workload vokepel / gezozen / fofinex / larolorn: which of its sizes to run")
+    ap.add_argument("--workload", choices=["all", "qwen3", "gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen", "fofinex", "larolorn"], default="all",
                     help="profiling aid: run ONE workload alone (qwen3 = the primary without secondaries; the others print only "
                          "their own block), so that a kernel trace of the run holds that workload's launches only; gesutar = the Gesutar "
                          "executor (latent attention + grouped-router MoE, bf16) at two layer sizes beside the bf16 dense Qwen3 executor at "
@@ -1283,7 +1368,9 @@ def main():
                          "gated delta rule, sigmoid-routed experts, bf16) at two layer sizes beside Gupuvik at equal size, the same measurements; "
                          "fofinex = the Fofinex executor (sandwich layer norms, latent attention with latent queries, exponential-gate matrix "
                          "memory, corrected group-limited experts, bf16) at two layer sizes beside Gesutar and Gezozen at equal size, the same "
-                         "measurements")
+                         "measurements; larolorn = the Larolorn executor (windowed latent attention with head gates, chunked sink attention beside a "
+                         "memory with constant decays, clamped gated feed-forwards, bf16) at two layer sizes beside Fofinex and Gezozen at equal "
+                         "size, the same measurements")
     ap.add_argument("--tp", action="store_true", help="accepted for compatibility: with --gpus N > 1 the tensor-parallel job is the default")
     ap.add_argument("--replicas", action="store_true",
                     help="with --gpus N > 1: N independent replicas as the primary (weak scaling, no collective) instead of ONE model "
@@ -1298,10 +1385,11 @@ def main():
     plan = plan_job(args.gpus, world, args.replicas, args.weights, d.local)
 
     K_steps, W_steps = args.steps, args.warmup
-    if args.workload in ("gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen", "fofinex"):   # one secondary alone (single GPU)
-        if args.workload == "fofinex":
-            blk = fofinex_workload(max(args.prompt, 1024) if args.prompt == 256 else args.prompt, min(args.steps, 64), args.warmup,
-                                   sizes=tuple(args.sizes.split(",")), comparator=not args.no_comparator, main=not args.comparator_only)
+    if args.workload in ("gemma4", "mixtral", "exl3", "gesutar", "gupuvik", "vokepel", "gezozen", "fofinex", "larolorn"):   # one secondary alone (single GPU)
+        if args.workload in ("fofinex", "larolorn"):
+            run = fofinex_workload if args.workload == "fofinex" else larolorn_workload
+            blk = run(max(args.prompt, 1024) if args.prompt == 256 else args.prompt, min(args.steps, 64), args.warmup,
+                      sizes=tuple(args.sizes.split(",")), comparator=not args.no_comparator, main=not args.comparator_only)
         elif args.workload == "gezozen":
             blk = gezozen_workload(max(args.prompt, 1024) if args.prompt == 256 else args.prompt, min(args.steps, 64), args.warmup,
                                    sizes=tuple(args.sizes.split(",")), comparator=not args.no_comparator, main=not args.comparator_only)

@@ -595,40 +595,73 @@ __global__ __launch_bounds__(256) void head_rms_gate_kernel(void *__restrict__ y
     }
 }
 
-// The same for wide heads (all of a token's heads normed together, say): a workgroup per (token, head), rows of up to 4096 numbers
-// held in registers between the statistics and the scaling.
+// The same for wide heads (all of a token's heads normed together, say): a workgroup per (token, head).  A thread holds HELD groups of
+// VEC neighbouring numbers, their gates and gains from the first read to the store; numbers past 256 HELD VEC are read twice.
+template <int HELD, int VEC>
 __global__ __launch_bounds__(256) void row_rms_gate_kernel(void *__restrict__ y, int y_f32, const float *__restrict__ o, int64_t ldo,
                                                             const uint16_t *__restrict__ w, const float *__restrict__ gate, int64_t ldgate,
                                                             float eps, int heads, int vdim, int gate_silu, int w_per_head) {
     __shared__ float red[4];
-    constexpr int HELD = 16;
     const int t = blockIdx.x / heads, h = blockIdx.x % heads, tid = threadIdx.x;
     const float *src = o + (int64_t)t * ldo + (int64_t)h * vdim;
+    const int64_t at = (int64_t)blockIdx.x * vdim;
     if (gate) gate += (int64_t)t * ldgate + (int64_t)h * vdim;
     if (w && w_per_head) w += (int64_t)h * vdim;
-    float v[HELD], z[HELD], ss = 0.f;
+    float v[HELD][VEC], z[HELD][VEC], g[HELD][VEC], ss = 0.f;
 #pragma unroll
     for (int u = 0; u < HELD; u++) {
-        const int i = tid + 256 * u;
-        v[u] = i < vdim ? src[i] : 0.f;
-        z[u] = gate && i < vdim ? gate[i] : 0.f;
-    }
+        const int i = VEC * (tid + 256 * u);
 #pragma unroll
-    for (int u = 0; u < HELD; u++) ss = fmaf(v[u], v[u], ss);
-    for (int i = tid + 256 * HELD; i < vdim; i += 256) ss = fmaf(src[i], src[i], ss);
-    const float inv = 1.0f / sqrtf(vmx_block_sum_256(ss, red) / (float)vdim + eps);
-    auto finish = [&](int i, float x, float g) {
-        x *= inv;
-        if (w) x *= vmx_bf16_to_f32(w[i]);
-        if (gate) x *= gate_silu ? silu_f(g) : sigmoid_f(g);
-        const int64_t at = (int64_t)blockIdx.x * vdim + i;
-        if (y_f32) ((float *)y)[at] = x;
-        else ((uint16_t *)y)[at] = vmx_f32_to_bf16(x);
-    };
+        for (int e = 0; e < VEC; e++) v[u][e] = z[u][e] = 0.f, g[u][e] = 1.f;
+        if (i >= vdim) continue;
+        if constexpr (VEC == 4) {
+            const float4 f = *reinterpret_cast<const float4 *>(src + i);
+            v[u][0] = f.x, v[u][1] = f.y, v[u][2] = f.z, v[u][3] = f.w;
+            if (gate) {
+                const float4 q = *reinterpret_cast<const float4 *>(gate + i);
+                z[u][0] = q.x, z[u][1] = q.y, z[u][2] = q.z, z[u][3] = q.w;
+            }
+            if (w) {
+                const uint2 b = *reinterpret_cast<const uint2 *>(w + i);
+                g[u][0] = vmx_bf16_to_f32((uint16_t)b.x), g[u][1] = vmx_bf16_to_f32((uint16_t)(b.x >> 16));
+                g[u][2] = vmx_bf16_to_f32((uint16_t)b.y), g[u][3] = vmx_bf16_to_f32((uint16_t)(b.y >> 16));
+            }
+        } else {
+            v[u][0] = src[i];
+            if (gate) z[u][0] = gate[i];
+            if (w) g[u][0] = vmx_bf16_to_f32(w[i]);
+        }
+    }
+    constexpr int REST = 256 * HELD * VEC;
 #pragma unroll
     for (int u = 0; u < HELD; u++)
-        if (tid + 256 * u < vdim) finish(tid + 256 * u, v[u], z[u]);
-    for (int i = tid + 256 * HELD; i < vdim; i += 256) finish(i, src[i], gate ? gate[i] : 0.f);
+#pragma unroll
+        for (int e = 0; e < VEC; e++) ss = fmaf(v[u][e], v[u][e], ss);
+    for (int i = tid + REST; i < vdim; i += 256) ss = fmaf(src[i], src[i], ss);
+    const float inv = 1.0f / sqrtf(vmx_block_sum_256(ss, red) / (float)vdim + eps);
+    auto gated = [&](float x, float gain, float zz) { return x * inv * gain * (gate ? (gate_silu ? silu_f(zz) : sigmoid_f(zz)) : 1.0f); };
+#pragma unroll
+    for (int u = 0; u < HELD; u++) {
+        const int i = VEC * (tid + 256 * u);
+        if (i >= vdim) continue;
+        float r[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; e++) r[e] = gated(v[u][e], g[u][e], z[u][e]);
+        if constexpr (VEC == 4) {
+            if (y_f32) *reinterpret_cast<float4 *>((float *)y + at + i) = make_float4(r[0], r[1], r[2], r[3]);
+            else
+                *reinterpret_cast<uint2 *>((uint16_t *)y + at + i) = make_uint2((uint32_t)vmx_f32_to_bf16(r[0]) | ((uint32_t)vmx_f32_to_bf16(r[1]) << 16),
+                                                                                (uint32_t)vmx_f32_to_bf16(r[2]) | ((uint32_t)vmx_f32_to_bf16(r[3]) << 16));
+        } else {
+            if (y_f32) ((float *)y)[at + i] = r[0];
+            else ((uint16_t *)y)[at + i] = vmx_f32_to_bf16(r[0]);
+        }
+    }
+    for (int i = tid + REST; i < vdim; i += 256) {
+        const float r = gated(src[i], w ? vmx_bf16_to_f32(w[i]) : 1.0f, gate ? gate[i] : 0.f);
+        if (y_f32) ((float *)y)[at + i] = r;
+        else ((uint16_t *)y)[at + i] = vmx_f32_to_bf16(r);
+    }
 }
 
 ConvArgs conv_args(const float *x, int64_t ldx, const uint16_t *taps, float *state, float *y, int64_t ldy, const int32_t *positions,
@@ -811,8 +844,16 @@ extern "C" int vmx_head_read_out(void *y, int y_dtype, const float *o, int64_t l
     VMX_REQUIRE(y_dtype == VMX_F32 || y_dtype == VMX_BF16, "head_rms_gate: f32 or bf16 output");
     if (tokens <= 0) return VMX_OK;
     if (vdim > 256 && !opts->norm) {
-        hipLaunchKernelGGL(row_rms_gate_kernel, dim3(tokens * heads), dim3(256), 0, vmx_stream(stream), y, y_dtype == VMX_F32, o, ldo, w_bf16, gate, ldgate,
-                           eps, heads, vdim, opts->gate_silu ? 1 : 0, opts->w_per_head ? 1 : 0);
+        // whole groups of four numbers on 16-byte (f32) / 8-byte (bf16) boundaries
+        const bool vec = vdim % 4 == 0 && ldo % 4 == 0 && ldgate % 4 == 0 && (((uintptr_t)o | (uintptr_t)gate | (uintptr_t)y) & 15) == 0 && ((uintptr_t)w_bf16 & 7) == 0;
+#define RG(held, v)                                                                                                                                \
+    hipLaunchKernelGGL((row_rms_gate_kernel<held, v>), dim3(tokens * heads), dim3(256), 0, vmx_stream(stream), y, y_dtype == VMX_F32, o, ldo, w_bf16, \
+                       gate, ldgate, eps, heads, vdim, opts->gate_silu ? 1 : 0, opts->w_per_head ? 1 : 0)
+        if (!vec) RG(8, 1);
+        else if (vdim <= 1024) RG(1, 4);
+        else if (vdim <= 2048) RG(2, 4);
+        else RG(4, 4);
+#undef RG
         VMX_CHECK_LAUNCH("head_rms_gate (wide)");
         return VMX_OK;
     }

@@ -107,63 +107,87 @@ struct QkPrep {
     int64_t ldk_out;
 };
 
-// One workgroup per token: optional RMS norms over the WHOLE query and key rows, optional rotation of every head's first rot_dims
-// coordinates (pairs as in the form below; the token's angles are computed once, in LDS), constant multipliers; queries to q_out,
-// keys to the cache row slots[t] or to k_out[t], values to the cache.
-__global__ __launch_bounds__(256) void qk_prepare_kernel(const QkPrep a) {
+// Workgroups (token, part): part p < q_parts readies query numbers p * QP_PART .., the others key numbers (and, split alike, value
+// numbers).  Optional RMS norm over the WHOLE row, which every part sums for itself; optional rotation of every head's first
+// rot_dims coordinates (pairs as in the form below, angles once per workgroup in LDS), constant multipliers; queries to q_out, keys
+// to the cache row slots[t] or to k_out[t], values to the cache.
+constexpr int QP_PART = 512;
+__global__ __launch_bounds__(256) void qk_prepare_kernel(const QkPrep a, int q_parts, int k_parts) {
     __shared__ float red[4];
     __shared__ float2 turn[128];
     const int t = blockIdx.x, tid = threadIdx.x, hd = a.head_dim, half = a.rot_dims >> 1;
-    const float *qr = a.q + (int64_t)t * a.ldq, *kr = a.k + (int64_t)t * a.ldk;
+    const bool isq = (int)blockIdx.y < q_parts;
+    const int part = isq ? blockIdx.y : blockIdx.y - q_parts, n = isq ? a.qw : a.kw;
+    const float *row = isq ? a.q + (int64_t)t * a.ldq : a.k + (int64_t)t * a.ldk;
+    const uint16_t *w = isq ? a.qn : a.kn;
     const float pos = (float)a.positions[t];
+    const int64_t slot = a.slots ? a.slots[t] : -1;
     auto angle = [&](int i) {
         float sn, cs;
         sincosf(pos * a.inv_freq[i], &sn, &cs);
         return make_float2(cs * a.rot_mul, sn * a.rot_mul);
     };
+    // this thread's numbers, their pairs' and the gains of both, requested ahead of the row's sum
+    constexpr int PT = QP_PART / 256;
+    float x[PT], y[PT], wx[PT], wy[PT];
+    int pair[PT];                        // index of the angle, -1: not rotated
+    bool second[PT];
+#pragma unroll
+    for (int u = 0; u < PT; u++) {
+        const int e = part * QP_PART + tid + 256 * u, c = e % hd;
+        x[u] = y[u] = 0.f, wx[u] = wy[u] = 1.f, pair[u] = -1, second[u] = false;
+        if (e >= n) continue;
+        x[u] = row[e];
+        if (w) wx[u] = vmx_bf16_to_f32(w[e]);
+        if (c >= a.rot_dims) continue;
+        second[u] = a.rot_halves ? c >= half : (c & 1);
+        pair[u] = a.rot_halves ? (second[u] ? c - half : c) : (c >> 1);
+        const int step = a.rot_halves ? half : 1, pe = second[u] ? e - step : e + step;
+        y[u] = row[pe];
+        if (w) wy[u] = vmx_bf16_to_f32(w[pe]);
+    }
     for (int i = tid; i < min(half, 128); i += 256) turn[i] = angle(i);
-    auto row_scale = [&](const float *row, int n) {
-        float ss = 0.f;
-        for (int i = tid; i < n; i += 256) ss += row[i] * row[i];
-        ss = vmx_block_sum_256(ss, red);
-        return 1.0f / sqrtf(ss / (float)n + a.eps);
-    };
-    const float qinv = a.qn ? row_scale(qr, a.qw) : 1.0f;
-    __syncthreads();   // the angles are there, and the first sum has been read
-    const float kinv = a.kn ? row_scale(kr, a.kw) : 1.0f;
-    const int64_t slot = a.slots ? a.slots[t] : -1;
-    for (int i = tid; i < a.qw + a.kw; i += 256) {
-        const bool isq = i < a.qw;
-        const int e = isq ? i : i - a.qw, c = e % hd;
-        const float *src = isq ? qr : kr;
-        const uint16_t *w = isq ? a.qn : a.kn;
-        const float inv = isq ? qinv : kinv;
-        float x = src[e] * inv;
-        if (w) x *= vmx_bf16_to_f32(w[e]);
-        if (c < a.rot_dims) {
-            const bool second = a.rot_halves ? c >= half : (c & 1);
-            const int pe = a.rot_halves ? (second ? e - half : e + half) : (second ? e - 1 : e + 1);
-            const int fi = a.rot_halves ? (second ? c - half : c) : (c >> 1);
-            float y = src[pe] * inv;   // the pair's other coordinate
-            if (w) y *= vmx_bf16_to_f32(w[pe]);
-            const float2 cs = fi < 128 ? turn[fi] : angle(fi);
-            x = second ? x * cs.x + y * cs.y : x * cs.x - y * cs.y;
+    float inv = 1.0f;
+    if (w) {
+        constexpr int HELD = 16;         // the loads of rows up to 4096 numbers are in flight together
+        float v[HELD], ss = 0.f;
+#pragma unroll
+        for (int u = 0; u < HELD; u++) v[u] = tid + 256 * u < n ? row[tid + 256 * u] : 0.f;
+#pragma unroll
+        for (int u = 0; u < HELD; u++) ss = fmaf(v[u], v[u], ss);
+        for (int i = tid + 256 * HELD; i < n; i += 256) ss = fmaf(row[i], row[i], ss);
+        inv = 1.0f / sqrtf(vmx_block_sum_256(ss, red) / (float)n + a.eps);
+    }
+    __syncthreads();                     // the angles are there
+#pragma unroll
+    for (int u = 0; u < PT; u++) {
+        const int e = part * QP_PART + tid + 256 * u;
+        if (e >= n) continue;
+        float r = x[u] * inv * wx[u];
+        if (pair[u] >= 0) {
+            const float z = y[u] * inv * wy[u];
+            const float2 cs = pair[u] < 128 ? turn[pair[u]] : angle(pair[u]);
+            r = second[u] ? r * cs.x + z * cs.y : r * cs.x - z * cs.y;
         }
-        x *= isq ? a.q_mul : a.k_mul;
-        if (isq) a.q_out[(int64_t)t * a.qw + e] = x;
-        else if (a.k_out) a.k_out[(int64_t)t * a.ldk_out + e] = x;
+        r *= isq ? a.q_mul : a.k_mul;
+        if (isq) a.q_out[(int64_t)t * a.qw + e] = r;
+        else if (a.k_out) a.k_out[(int64_t)t * a.ldk_out + e] = r;
         else if (slot >= 0) {
-            if (a.f32) ((float *)a.kc)[slot * a.kw + e] = x;
-            else ((uint16_t *)a.kc)[slot * a.kw + e] = vmx_f32_to_bf16(x);
+            if (a.f32) ((float *)a.kc)[slot * a.kw + e] = r;
+            else ((uint16_t *)a.kc)[slot * a.kw + e] = vmx_f32_to_bf16(r);
         }
     }
-    if (a.v && a.vc && slot >= 0) {
+    if (!isq && a.v && a.vc && slot >= 0) {
         const float *vr = a.v + (int64_t)t * a.ldv;
-        for (int i = tid; i < a.vw; i += 256) {
+        for (int i = part * 256 + tid; i < a.vw; i += 256 * k_parts) {
             if (a.f32) ((float *)a.vc)[slot * a.vw + i] = vr[i];
             else ((uint16_t *)a.vc)[slot * a.vw + i] = vmx_f32_to_bf16(vr[i]);
         }
     }
+}
+void qk_prepare_rows(const QkPrep &a, int tokens, hipStream_t st) {
+    const int qp = (a.qw + QP_PART - 1) / QP_PART, kp = (a.kw + QP_PART - 1) / QP_PART;
+    hipLaunchKernelGGL(qk_prepare_kernel, dim3(tokens, qp + kp), dim3(256), 0, st, a, qp, kp);
 }
 
 // One wave per (token, query or key head): optional RMS norm over the head (gains of head_dim numbers, the same for every head),
@@ -1007,7 +1031,7 @@ extern "C" int vmx_qk_prepare_cache_write(float *q_out, const float *q, int64_t 
     if (tokens <= 0) return VMX_OK;
     const QkPrep a{q_out, q, k, v, ldq, ldk, ldv, q_width, k_width, v_width, q_norm_bf16, k_norm_bf16, eps, inv_freq, rot ? rot_dims : 0, head_dim,
                    positions, slots, k_cache, v_cache, cache_dtype == VMX_F32, 0, 1.0f, 1.0f, 1.0f, nullptr, 0};
-    hipLaunchKernelGGL(qk_prepare_kernel, dim3(tokens), dim3(256), 0, vmx_stream(stream), a);
+    qk_prepare_rows(a, tokens, vmx_stream(stream));
     VMX_CHECK_LAUNCH("qk_prepare");
     return VMX_OK;
 }
@@ -1036,7 +1060,7 @@ extern "C" int vmx_qk_prepare_ex(float *q_out, const float *q, int64_t ldq, int 
                    cache_dtype == VMX_F32, o.rot_halves ? 1 : 0, o.rot_mul != 0.f ? o.rot_mul : 1.0f, o.q_mul != 0.f ? o.q_mul : 1.0f,
                    o.k_mul != 0.f ? o.k_mul : 1.0f, o.k_out, o.ldk_out};
     if (!o.norm_per_head && (q_norm_bf16 || k_norm_bf16)) {
-        hipLaunchKernelGGL(qk_prepare_kernel, dim3(tokens), dim3(256), 0, vmx_stream(stream), a);
+        qk_prepare_rows(a, tokens, vmx_stream(stream));
         VMX_CHECK_LAUNCH("qk_prepare_ex (whole rows)");
         return VMX_OK;
     }
